@@ -55,5 +55,9 @@ from .lurisun import LurisunRingModel  # noqa: E402
 
 register(LurisunRingModel)
 
+from .turevik import TurevikRingModel  # noqa: E402
+
+register(TurevikRingModel)
+
 __all__ = ["GegoraxRingModel", "KomizenRingModel", "LurisunRingModel", "ModelConfig", "QuantConfig", "RingModel", "MoERingModel", "KVCache", "PosudraRingModel",
-           "Linear", "PRESETS", "get_ring_model", "register"]
+           "TurevikRingModel", "Linear", "PRESETS", "get_ring_model", "register"]

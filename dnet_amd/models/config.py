@@ -351,8 +351,88 @@ class ModelConfig:
         )
 
     @classmethod
+    def from_turevik(cls, cfg: dict,
+                     quant: Optional[QuantConfig] = None) -> "ModelConfig":
+        """Turevik checkpoints list their layers: {"architecture":
+        "Turevik", "vocab", "width", "norm": {"eps"}, "layers": [{"type":
+        "latent_attention" | "mingru", "mixer": {...}, "mlp": {"kind":
+        "dense", "ff"} | {"kind": "moe", "router": {"experts", "top"},
+        "expert": {"ff"}, "shared": {"ff"} (optional)} | null}, ...]}. A
+        latent-attention mixer with "kv_from": j reads the cached rows of the
+        earlier layer j. Every size is per layer."""
+        need = {"mingru": ("width",),
+                "latent_attention": ("dim", "heads", "kv_rank", "rot",
+                                     "rot_dim", "scale", "vdim")}
+        specs = [dict(s) for s in cfg["layers"]]
+        for i, s in enumerate(specs):
+            kind, m = s.get("type"), s.get("mixer") or {}
+            if kind not in need:
+                raise ValueError(f"turevik layer {i}: unknown mixer type "
+                                 f"{kind!r}")
+            missing = [k for k in need[kind] if k not in m]
+            if missing:
+                raise ValueError(f"turevik layer {i}: mixer lacks {missing}")
+            if kind == "latent_attention":
+                if int(m["rot"]["dims"]) != int(m["rot_dim"]) \
+                        or int(m["rot_dim"]) % 2:
+                    raise ValueError(f"turevik layer {i}: rot.dims must be "
+                                     "the (even) rotated size")
+                j = m.get("kv_from")
+                if j is not None:
+                    o = specs[j] if 0 <= j < i else {}
+                    om = o.get("mixer") or {}
+                    if o.get("type") != kind or om.get("kv_from") is not None:
+                        raise ValueError(f"turevik layer {i}: kv_from must "
+                                         "name an earlier layer with rows of "
+                                         "its own")
+                    if any(om[k] != m[k] for k in ("kv_rank", "rot_dim",
+                                                   "rot")):
+                        raise ValueError(f"turevik layer {i}: kv_rank and "
+                                         "rotation differ from layer "
+                                         f"{j}'s")
+            ff = s.get("mlp")
+            if ff is not None:
+                if ff.get("kind") not in ("dense", "moe"):
+                    raise ValueError(f"turevik layer {i}: unknown "
+                                     f"feed-forward kind {ff.get('kind')!r}")
+                if ff["kind"] == "moe" and not (
+                        0 < ff["router"]["top"] <= ff["router"]["experts"]):
+                    raise ValueError(f"turevik layer {i}: router.top")
+        att = next((s["mixer"] for s in specs
+                    if s["type"] == "latent_attention"), {})
+        ffs = [s["mlp"] for s in specs if s.get("mlp") is not None]
+        moe = [f for f in ffs if f["kind"] == "moe"]
+        return cls(
+            model_type="turevik",
+            hidden_size=cfg["width"],
+            num_layers=len(specs),
+            num_q_heads=att.get("heads", 1),
+            num_kv_heads=1,
+            head_dim=att.get("dim", 1),
+            v_head_dim=att.get("vdim", 1),
+            kv_lora_rank=att.get("kv_rank", 0),
+            intermediate_size=max((f["ff"] for f in ffs
+                                   if f["kind"] == "dense"), default=0),
+            num_experts=max((f["router"]["experts"] for f in moe), default=0),
+            num_experts_per_tok=max((f["router"]["top"] for f in moe),
+                                    default=0),
+            moe_intermediate_size=max((f["expert"]["ff"] for f in moe),
+                                      default=0),
+            shared_expert_intermediate_size=max(
+                (f["shared"]["ff"] for f in moe if f.get("shared")),
+                default=0),
+            vocab_size=cfg["vocab"],
+            rms_eps=cfg["norm"]["eps"],
+            tie_word_embeddings=True,
+            layer_specs=specs,
+            quant=quant,
+        )
+
+    @classmethod
     def from_hf(cls, cfg: dict, quant: Optional[QuantConfig] = None) -> "ModelConfig":
         arch = str(cfg.get("architecture", "")).lower()
+        if arch == "turevik" or cfg.get("model_type") == "turevik":
+            return cls.from_turevik(cfg, quant)
         if arch == "lurisun" or cfg.get("model_type") == "lurisun":
             return cls.from_lurisun(cfg, quant)
         if arch == "posudra" or cfg.get("model_type") == "posudra":
@@ -562,6 +642,46 @@ def lurisun_config(width: int, vocab: int, pattern: str = "nla",
     return cfg
 
 
+def turevik_config(width: int, vocab: int, pattern: str = "lsg",
+                   layers: int = 0, heads: int = 4, dim: int = 32,
+                   rot_dim: int = 16, vdim: int = 32, kv_rank: int = 64,
+                   gru_width: int = 0, ff: int = 192, dense_every: int = 0,
+                   experts: int = 4, top: int = 2, expert_ff: int = 64,
+                   shared_ff: int = 48, rot_base: float = 10000.0,
+                   eps: float = 1e-6) -> dict:
+    """A turevik stack in the checkpoint's config.json layout. ``pattern``
+    repeats over ``layers`` layers (default: once): 'l' = latent attention
+    with rows of its own, 's' = latent attention on the rows of the nearest
+    earlier 'l', 'g' = minGRU (``gru_width`` channels, 0 = the model width).
+    Feed-forwards: layer 0 dense (and every ``dense_every``-th layer, 0 =
+    layer 0 only), mixtures of experts otherwise; no experts = all dense."""
+    out, own = [], None
+    for i in range(layers or len(pattern)):
+        c = pattern[i % len(pattern)]
+        if c == "g":
+            kind, m = "mingru", {"width": gru_width or width}
+        else:
+            kind = "latent_attention"
+            m = {"heads": heads, "dim": dim, "rot_dim": rot_dim,
+                 "vdim": vdim, "kv_rank": kv_rank,
+                 "scale": (dim + rot_dim) ** -0.5,
+                 "rot": {"base": rot_base, "dims": rot_dim}}
+            if c == "l":
+                own = i
+            else:
+                m["kv_from"] = own
+        if not experts or i == 0 or (dense_every and i % dense_every == 0):
+            mlp = {"kind": "dense", "ff": ff} if ff else None
+        else:
+            mlp = {"kind": "moe", "expert": {"ff": expert_ff},
+                   "router": {"experts": experts, "top": top}}
+            if shared_ff:
+                mlp["shared"] = {"ff": shared_ff}
+        out.append({"type": kind, "mixer": m, "mlp": mlp})
+    return {"architecture": "Turevik", "vocab": vocab, "width": width,
+            "norm": {"eps": eps}, "layers": out}
+
+
 # Known configs for synthetic benchmarking (random-init weights; no network).
 PRESETS: dict[str, dict] = {
     "llama-3-8b": dict(model_type="llama", hidden_size=4096, num_hidden_layers=32,
@@ -631,6 +751,7 @@ PRESETS: dict[str, dict] = {
                                    embedding_scale=4.0),
     "lurisun-tiny": lurisun_config(128, 256, "nla", layers=4,
                                    logit_scale=0.5),
+    "turevik-tiny": turevik_config(128, 256, "lsgs", layers=4),
     "tiny": dict(model_type="llama", hidden_size=128, num_hidden_layers=4,
                  num_attention_heads=2, num_key_value_heads=2, head_dim=64,
                  intermediate_size=256, vocab_size=256, rope_theta=10000.0),

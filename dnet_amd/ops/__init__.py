@@ -866,3 +866,152 @@ def mul_sigmoid(a, gate_src, col0: int) -> torch.Tensor:
         _native().mul_sigmoid(a.contiguous(), gate_src, col0, y)
         return y
     return ref.mul_sigmoid(a, gate_src, col0)
+
+
+# ---- token shift, minGRU, sigmoid-routed experts with scaled inputs
+# (turevik) ----
+# csrc/token_shift.hip.cpp, csrc/moe_rows.hip.cpp. Norms, the shift, the
+# recurrence with its gates and the router are fp32 whatever the activation
+# dtype.
+
+def norm_token_shift(x, wn, mu, prev, pos, T: int, eps: float,
+                     out_dtype: torch.dtype, lens=None,
+                     slots=None) -> torch.Tensor:
+    """h = rms(x) * wn, then h + (h' - h) * mu with the previous token's h
+    (``prev`` fp32 [Bc, W]: each slot's last h, read and advanced)."""
+    if x.is_cuda:
+        y = torch.empty(x.shape, dtype=out_dtype, device=x.device)
+        _native().norm_token_shift(x, None, None, wn, mu, prev, y, pos, lens,
+                                   slots, T, eps)
+        return y
+    return ref.norm_token_shift(x, wn, mu, prev, pos, T, eps, out_dtype, lens,
+                                slots)
+
+
+def resid_norm_token_shift(x, a, wa, wn, mu, prev, pos, T: int, eps: float,
+                           out_dtype: torch.dtype, lens=None,
+                           slots=None) -> torch.Tensor:
+    """x (fp32, in place) += rms(a) * wa, then ``norm_token_shift`` of it:
+    one kernel in decode steps, two for prompts (a token's shift there reads
+    the updated residual of the row before it)."""
+    if x.is_cuda:
+        y = torch.empty(x.shape, dtype=out_dtype, device=x.device)
+        if T == 1:
+            _native().norm_token_shift(x, a, wa, wn, mu, prev, y, pos, lens,
+                                       slots, T, eps)
+        else:
+            _native().resid_branches_rmsnorm(x, a, wa, None, None, 1.0, None,
+                                             None, None, None, eps)
+            _native().norm_token_shift(x, None, None, wn, mu, prev, y, pos,
+                                       lens, slots, T, eps)
+        return y
+    return ref.resid_norm_token_shift(x, a, wa, wn, mu, prev, pos, T, eps,
+                                      out_dtype, lens, slots)
+
+
+def mingru_scan(src, z0: int, x0: int, g0: int, bz, bx, state, pos, T: int,
+                lens=None, slots=None) -> torch.Tensor:
+    """S <- (1 - z) S + z * candidate per channel (fp32 state [Bc, N]); the
+    result S * silu(gate) in src's dtype."""
+    if src.is_cuda:
+        # padded rows of a ragged batch are never written by the kernel
+        y = (torch.zeros if lens is not None else torch.empty)(
+            src.shape[0], bz.numel(), dtype=src.dtype, device=src.device)
+        _native().mingru_scan(src, z0, x0, g0, bz, bx, state, y, pos, lens,
+                              slots, T)
+        return y
+    return ref.mingru_scan(src, z0, x0, g0, bz, bx, state, pos, T, lens,
+                           slots)
+
+
+def cache_append(src, col0: int, cache, pos, T: int, lens=None,
+                 slots=None) -> None:
+    """Columns of src as they are into cache rows (see the reference)."""
+    if src.is_cuda:
+        _native().cache_append(src, col0, cache, pos, lens, slots, T)
+        return
+    ref.cache_append(src, col0, cache, pos, T, lens, slots)
+
+
+_GATED_ACTS = {"silu": 0, "gelu_tanh": 1}
+
+
+def gated_act(gu, act: str, scale=None) -> torch.Tensor:
+    """[gate | up] -> act(s gate) * (s up), s the row's ``scale`` (or 1)."""
+    if gu.is_cuda:
+        y = torch.empty(gu.shape[0], gu.shape[1] // 2, dtype=gu.dtype,
+                        device=gu.device)
+        _native().gated_act(gu, scale, y, _GATED_ACTS[act])
+        return y
+    return ref.gated_act(gu, act, scale)
+
+
+# rows up to which the router's products run inside the routing kernel
+_ROUTER_FUSED_ROWS = 128
+
+
+def moe_router(x, w, E: int, top: int):
+    """Sigmoid router in fp32 with an optional shared-expert gate as the last
+    row of w [E (+1), W]: (idx, val, we, gate), see the reference. No host
+    sync."""
+    if x.is_cuda:
+        T = x.shape[0]
+        idx = torch.empty(T, top, dtype=torch.int32, device=x.device)
+        val = torch.empty(T, top, dtype=torch.float32, device=x.device)
+        we = torch.empty(T, E, dtype=torch.float32, device=x.device)
+        gate = (torch.empty(T, dtype=torch.float32, device=x.device)
+                if w.shape[0] > E else None)
+        if T <= _ROUTER_FUSED_ROWS:
+            _native().moe_router(x, w, None, idx, val, we, gate)
+        else:
+            _native().moe_router(None, None, x.float() @ w.t(), idx, val, we,
+                                 gate)
+        return idx, val, we, gate
+    return ref.moe_router(x, w, E, top)
+
+
+def moe_plan(idx, E: int):
+    """Entries (t, k) of idx [T, top] grouped by expert: (order, at, counts),
+    see the reference."""
+    if idx.is_cuda:
+        order = torch.empty(idx.numel(), dtype=torch.int32, device=idx.device)
+        at = torch.empty_like(idx)
+        counts = torch.empty(E, dtype=torch.int32, device=idx.device)
+        _native().moe_plan(idx, order, at, counts)
+        return order, at, counts
+    return ref.moe_plan(idx, E)
+
+
+def moe_gateup_rows(x, w, we) -> torch.Tensor:
+    """bf16 experts on the matrix cores for decode-sized batches: act [E, T,
+    I] = silu(we gate) * (we up); experts no row chose are skipped on the
+    device (their act is not written)."""
+    if x.is_cuda:
+        E, I2, _ = w.shape
+        act = torch.empty(E, x.shape[0], I2 // 2, dtype=x.dtype,
+                          device=x.device)
+        _native().moe_gateup_rows(x, w, we, act)
+        return act
+    return ref.moe_gateup_rows(x, w, we)
+
+
+def moe_down_rows(act, w, we) -> torch.Tensor:
+    """Second half of ``moe_gateup_rows``: [E, T, N], skipped experts
+    unwritten; ``moe_merge`` reads the chosen ones only."""
+    if act.is_cuda:
+        y = torch.empty(act.shape[0], act.shape[1], w.shape[1],
+                        dtype=act.dtype, device=act.device)
+        _native().moe_down_rows(act, w, we, y)
+        return y
+    return ref.moe_down_rows(act, w, we)
+
+
+def moe_merge(y, at, shared, gate, out_dtype: torch.dtype) -> torch.Tensor:
+    """Sum of each row's chosen results (+ gate * shared), fp32 sum, one
+    rounding. See the reference for y / at."""
+    if y.is_cuda:
+        out = torch.empty(at.shape[0], y.shape[-1], dtype=out_dtype,
+                          device=y.device)
+        _native().moe_merge(y, at, shared, gate, out)
+        return out
+    return ref.moe_merge(y, at, shared, gate, out_dtype)

@@ -1023,8 +1023,9 @@ def latent_append(src: torch.Tensor, col0: int, wn: torch.Tensor, eps: float,
 def latent_q_pack(q: torch.Tensor, qabs: torch.Tensor,
                   rot_freq: torch.Tensor, pos: torch.Tensor, T: int, H: int,
                   d: int) -> torch.Tensor:
-    """Queries of latent attention in the cache's layout. q [B*T, H*(d+rd)]
-    holds per head d plain and rd turning dimensions; qabs [H, B*T, R] the
+    """Queries of latent attention in the cache's layout. q [B*T, >=
+    H*(d+rd)] holds per head d plain and rd turning dimensions (columns
+    after those are ignored); qabs [H, B*T, R] the
     plain part already carried into the latent space. Returns [B*T,
     H*(R+rd)] = per head [qabs | turned part] (angles as in
     ``latent_append``)."""
@@ -1035,7 +1036,8 @@ def latent_q_pack(q: torch.Tensor, qabs: torch.Tensor,
     tpos = (pos.to(torch.int64).view(B, 1)
             + torch.arange(T, device=q.device)).reshape(M).to(torch.float32)
     ang = tpos.view(M, 1) * rot_freq.float().view(1, -1)
-    qr = rotate_pairs(q.view(M, H, d + rd)[..., d:].float(), ang)
+    qr = rotate_pairs(q[:, :H * (d + rd)].reshape(M, H, d + rd)[..., d:]
+                      .float(), ang)
     out = torch.cat([qabs.transpose(0, 1).float(), qr], dim=-1)
     return out.reshape(M, H * (R + rd)).to(q.dtype)
 
@@ -1214,3 +1216,165 @@ def mul_sigmoid(a: torch.Tensor, gate_src: torch.Tensor,
     N = a.shape[1]
     return (a.float() * torch.sigmoid(gate_src[:, col0:col0 + N].float())
             ).to(a.dtype)
+
+
+# ---- token shift, minGRU, sigmoid-routed experts with scaled inputs
+# (turevik) ----
+
+def norm_token_shift(x: torch.Tensor, wn: torch.Tensor, mu: torch.Tensor,
+                     prev: torch.Tensor, pos: torch.Tensor, T: int,
+                     eps: float, out_dtype: torch.dtype, lens=None,
+                     slots=None) -> torch.Tensor:
+    """RMS norm followed by a token shift. x fp32 [B*T, W]; h = rms(x) * wn;
+    y = h + (h' - h) * mu with h' the previous token's h (zero before
+    position 0). ``prev`` fp32 [Bc, W] holds each slot's last h and is
+    advanced by the rows' real tokens (t < lens[b])."""
+    M = x.shape[0]
+    B = M // T
+    h = rmsnorm_rows(x, wn, eps, torch.float32)
+    out = h.clone()
+    p, ln, sl = _row_index(B, T, pos, lens, slots, x.device)
+    for b in range(B):
+        n = int(min(ln[b], T))
+        if n <= 0:
+            continue
+        s = int(sl[b])
+        hb = h[b * T:b * T + n]
+        first = prev[s].view(1, -1) if int(p[b]) > 0 else \
+            torch.zeros_like(hb[:1])
+        before = torch.cat([first, hb[:-1]])
+        out[b * T:b * T + n] = hb + (before - hb) * mu
+        prev[s] = hb[-1]
+    return out.to(out_dtype)
+
+
+def resid_norm_token_shift(x, a, wa, wn, mu, prev, pos, T: int, eps: float,
+                           out_dtype: torch.dtype, lens=None, slots=None):
+    """x (fp32, in place) += rms(a) * wa, then ``norm_token_shift`` of it."""
+    resid_branches_rmsnorm(x, a, wa, None, None, 1.0, None, None, eps,
+                           out_dtype, False)
+    return norm_token_shift(x, wn, mu, prev, pos, T, eps, out_dtype, lens,
+                            slots)
+
+
+def mingru_scan(src: torch.Tensor, z0: int, x0: int, g0: int,
+                bz: torch.Tensor, bx: torch.Tensor, state: torch.Tensor,
+                pos: torch.Tensor, T: int, lens=None,
+                slots=None) -> torch.Tensor:
+    """Gated recurrence whose gates read the current token only, fp32. With
+    N = len(bz) and columns z0 / x0 / g0 of src [B*T, ld]: z = sigmoid(zc +
+    bz), u = xc + bx, candidate = u + 1/2 where u >= 0 and sigmoid(u)
+    elsewhere; S <- (1 - z) S + z * candidate; y = S * silu(gc), in src's
+    dtype. ``state`` fp32 [Bc, N] per slot: zero at position 0, advanced by
+    the rows' real tokens. Padding rows of y are zero."""
+    M, N = src.shape[0], bz.numel()
+    B = M // T
+    f = src.float()
+    z = torch.sigmoid(f[:, z0:z0 + N] + bz)
+    u = f[:, x0:x0 + N] + bx
+    c = torch.where(u >= 0, u + 0.5, torch.sigmoid(u))
+    gate = torch.nn.functional.silu(f[:, g0:g0 + N])
+    out = torch.zeros(M, N, dtype=torch.float32, device=src.device)
+    p, ln, sl = _row_index(B, T, pos, lens, slots, src.device)
+    for b in range(B):
+        n = int(min(ln[b], T))
+        if n <= 0:
+            continue
+        s = int(sl[b])
+        S = state[s].clone() if int(p[b]) > 0 else torch.zeros_like(state[s])
+        for t in range(b * T, b * T + n):
+            S = (1.0 - z[t]) * S + z[t] * c[t]
+            out[t] = S * gate[t]
+        state[s] = S
+    return out.to(src.dtype)
+
+
+def cache_append(src: torch.Tensor, col0: int, cache: torch.Tensor,
+                 pos: torch.Tensor, T: int, lens=None, slots=None) -> None:
+    """Columns [col0, col0 + H*D) of src [B*T, ld] as they are to cache
+    [Bc, H, Smax, D] at position pos[b]+t of row slots[b] (padding tokens are
+    not appended)."""
+    H, D = cache.shape[1], cache.shape[3]
+    B = src.shape[0] // T
+    p, ln, sl = _row_index(B, T, pos, lens, slots, src.device)
+    for b in range(B):
+        n = int(min(ln[b], T))
+        if n <= 0:
+            continue
+        p0, s = int(p[b]), int(sl[b])
+        cache[s, :, p0:p0 + n] = src[b * T:b * T + n, col0:col0 + H * D] \
+            .reshape(n, H, D).transpose(0, 1).to(cache.dtype)
+
+
+def gated_act(gu: torch.Tensor, act: str, scale=None) -> torch.Tensor:
+    """gu [M, 2I] = [gate | up] -> act(gate) * up [M, I], fp32 math.
+    ``scale`` fp32 [M]: factor of the row's input, act(s gate) * (s up)."""
+    i = gu.shape[-1] // 2
+    f = gu.float()
+    if scale is not None:
+        f = f * scale.view(-1, 1)
+    g, u = f[:, :i], f[:, i:]
+    g = (torch.nn.functional.gelu(g, approximate="tanh") if act == "gelu_tanh"
+         else torch.nn.functional.silu(g))
+    return (g * u).to(gu.dtype)
+
+
+def moe_router(x: torch.Tensor, w: torch.Tensor, E: int, top: int):
+    """Sigmoid router in fp32. x [T, W], w fp32 [E or E+1, W] (the last row,
+    when there, is the shared expert's gate). Returns (idx int32 [T, top],
+    val fp32 [T, top], we fp32 [T, E] with the values of the chosen experts
+    and 0 elsewhere, gate fp32 [T] or None)."""
+    z = torch.sigmoid(x.float() @ w.t())
+    val, idx = torch.topk(z[:, :E], top, dim=-1)
+    we = torch.zeros_like(z[:, :E]).scatter_(1, idx, val)
+    gate = z[:, E].contiguous() if w.shape[0] > E else None
+    return idx.to(torch.int32), val, we, gate
+
+
+def moe_merge(y: torch.Tensor, at: torch.Tensor, shared, gate,
+              out_dtype: torch.dtype) -> torch.Tensor:
+    """out[t] = sum_k y[at[t, k]] (+ gate[t] * shared[t]), summed in fp32.
+    y [R, W] and at int32 [T, top] its rows, or y [E, T, W] and at the
+    chosen experts (then row (at[t, k], t)); shared [T, W] and gate fp32 [T]
+    optional."""
+    at = at.long()
+    if y.dim() == 3:
+        at = at * y.shape[1] + torch.arange(at.shape[0],
+                                            device=at.device).view(-1, 1)
+        y = y.reshape(-1, y.shape[2])
+    out = y[at].float().sum(dim=1)
+    if shared is not None:
+        out = out + gate.view(-1, 1) * shared.float()
+    return out.to(out_dtype)
+
+
+def moe_plan(idx: torch.Tensor, E: int):
+    """Rows sorted by expert. idx int32 [T, top] -> (order int32 [T*top]: the
+    flat entries (t*top + k) expert by expert, entries of one expert in
+    ascending order; at int32 [T, top]: each entry's place in that order;
+    counts int32 [E])."""
+    flat = idx.reshape(-1).long()
+    order = torch.argsort(flat, stable=True)
+    at = torch.empty_like(order)
+    at[order] = torch.arange(flat.numel(), device=idx.device)
+    return (order.to(torch.int32), at.view(idx.shape).to(torch.int32),
+            torch.bincount(flat, minlength=E).to(torch.int32))
+
+
+def moe_gateup_rows(x: torch.Tensor, w: torch.Tensor,
+                    we: torch.Tensor) -> torch.Tensor:
+    """Experts' first half on every row, inputs scaled by the routing
+    weight: x [T, K], w [E, 2I, K], we [T, E] -> act [E, T, I] =
+    silu(we gate) * (we up) in x's dtype (0 for rows that did not choose the
+    expert)."""
+    z = torch.einsum("tk,eik->eti", x.float(), w.float())
+    z = z * we.t().unsqueeze(-1)
+    i = z.shape[-1] // 2
+    return (torch.nn.functional.silu(z[..., :i]) * z[..., i:]).to(x.dtype)
+
+
+def moe_down_rows(act: torch.Tensor, w: torch.Tensor,
+                  we: torch.Tensor) -> torch.Tensor:
+    """Experts' second half: act [E, T, I], w [E, N, I] -> [E, T, N] in
+    act's dtype (rows of experts nobody chose may hold anything)."""
+    return torch.einsum("eti,eni->etn", act.float(), w.float()).to(act.dtype)
