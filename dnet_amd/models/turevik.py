@@ -435,8 +435,7 @@ class TurevikRingModel(RingModel):
             return ops.moe_merge(y, idx, shared, gate, self.wdtype)
         # prompts: rows sorted by expert, one product per expert and half
         order, at, counts = ops.moe_plan(idx, E)
-        entry = order.long()
-        xs = u[entry // top]
+        xs, scale = ops.moe_gather(u, order, val)
         gu = torch.empty(M * top, 2 * I, dtype=u.dtype, device=u.device)
         y = torch.empty(M * top, W, dtype=u.dtype, device=u.device)
         n = counts.tolist()
@@ -444,7 +443,7 @@ class TurevikRingModel(RingModel):
         spans = [(e, ends[e] - n[e], ends[e]) for e in range(E) if n[e]]
         for e, a, b in spans:
             torch.mm(xs[a:b], lw.gateup_w[e].t(), out=gu[a:b])
-        act = ops.gated_act(gu, "silu", val.reshape(-1)[entry])
+        act = ops.gated_act(gu, "silu", scale)
         for e, a, b in spans:
             torch.mm(act[a:b], lw.down_w[e].t(), out=y[a:b])
         return ops.moe_merge(y, at, shared, gate, self.wdtype)

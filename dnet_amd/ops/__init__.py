@@ -982,6 +982,19 @@ def moe_plan(idx, E: int):
     return ref.moe_plan(idx, E)
 
 
+def moe_gather(x, order, val):
+    """Rows of x [T, W] and scales val [T, top] of the sorted entries
+    ``order``: (xs [T*top, W], scale fp32 [T*top])."""
+    if x.is_cuda:
+        xs = torch.empty(order.numel(), x.shape[1], dtype=x.dtype,
+                         device=x.device)
+        scale = torch.empty(order.numel(), dtype=torch.float32,
+                            device=x.device)
+        _native().moe_gather(x, order, val, xs, scale)
+        return xs, scale
+    return ref.moe_gather(x, order, val)
+
+
 def moe_gateup_rows(x, w, we) -> torch.Tensor:
     """bf16 experts on the matrix cores for decode-sized batches: act [E, T,
     I] = silu(we gate) * (we up); experts no row chose are skipped on the

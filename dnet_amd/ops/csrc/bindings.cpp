@@ -183,6 +183,37 @@ void moe_up_act(torch::Tensor x, torch::Tensor w, torch::Tensor we,
 void moe_route(torch::Tensor logits, torch::Tensor we, int64_t top,
                double scale);
 void moe_weighted_sum(torch::Tensor d, torch::Tensor we, torch::Tensor out);
+void norm_token_shift(torch::Tensor x, c10::optional<torch::Tensor> a,
+                      c10::optional<torch::Tensor> wa, torch::Tensor wn,
+                      torch::Tensor mu, torch::Tensor prev, torch::Tensor y,
+                      torch::Tensor pos, c10::optional<torch::Tensor> lens,
+                      c10::optional<torch::Tensor> slots, int64_t T,
+                      double eps);
+void mingru_scan(torch::Tensor src, int64_t z0, int64_t x0, int64_t g0,
+                 torch::Tensor bz, torch::Tensor bx, torch::Tensor state,
+                 torch::Tensor y, torch::Tensor pos,
+                 c10::optional<torch::Tensor> lens,
+                 c10::optional<torch::Tensor> slots, int64_t T);
+void cache_append(torch::Tensor src, int64_t col0, torch::Tensor cache,
+                  torch::Tensor pos, c10::optional<torch::Tensor> lens,
+                  c10::optional<torch::Tensor> slots, int64_t T);
+void gated_act(torch::Tensor gu, c10::optional<torch::Tensor> scale,
+               torch::Tensor y, int64_t kind);
+void moe_router(c10::optional<torch::Tensor> x, torch::Tensor w,
+                c10::optional<torch::Tensor> logits, torch::Tensor idx,
+                torch::Tensor val, torch::Tensor we,
+                c10::optional<torch::Tensor> gate);
+void moe_plan(torch::Tensor idx, torch::Tensor order, torch::Tensor at,
+              torch::Tensor counts);
+void moe_gather(torch::Tensor x, torch::Tensor order, torch::Tensor val,
+                torch::Tensor xs, torch::Tensor scale);
+void moe_gateup_rows(torch::Tensor x, torch::Tensor w, torch::Tensor we,
+                     torch::Tensor act);
+void moe_down_rows(torch::Tensor act, torch::Tensor w, torch::Tensor we,
+                   torch::Tensor y);
+void moe_merge(torch::Tensor y, torch::Tensor at,
+               c10::optional<torch::Tensor> shared,
+               c10::optional<torch::Tensor> gate, torch::Tensor out);
 }  // namespace dnet
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -288,4 +319,23 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "softmax over all experts, top-k kept, scaled, not renormalized");
   m.def("moe_weighted_sum", &dnet::moe_weighted_sum,
         "sum over experts of routing weight times expert result");
+  m.def("norm_token_shift", &dnet::norm_token_shift,
+        "(fp32 residual += normalized branch,) RMSNorm and token shift with "
+        "the previous token's norm as per-slot state");
+  m.def("mingru_scan", &dnet::mingru_scan,
+        "minGRU recurrence with its output gate");
+  m.def("cache_append", &dnet::cache_append,
+        "projection columns as they are into cache rows");
+  m.def("gated_act", &dnet::gated_act,
+        "act(s gate) * (s up), silu or tanh-gelu, optional row factor");
+  m.def("moe_router", &dnet::moe_router,
+        "sigmoid router: top-k scores kept as they are, shared-expert gate");
+  m.def("moe_plan", &dnet::moe_plan, "routed entries sorted by expert");
+  m.def("moe_gather", &dnet::moe_gather, "rows and scales of sorted entries");
+  m.def("moe_gateup_rows", &dnet::moe_gateup_rows,
+        "gated experts on a decode batch, inputs scaled (matrix cores)");
+  m.def("moe_down_rows", &dnet::moe_down_rows,
+        "experts' down projection on a decode batch (matrix cores)");
+  m.def("moe_merge", &dnet::moe_merge,
+        "sum of each row's chosen expert results + gate * shared");
 }

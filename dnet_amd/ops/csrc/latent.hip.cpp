@@ -62,10 +62,10 @@ __global__ __launch_bounds__(256) void latent_append_kernel(
   }
 }
 
-// grid (B*T); q [M, H*(d+rd)], qabs [H, M, R] -> out [M, H*(R+rd)]
+// grid (B*T); q [M, ld >= H*(d+rd)], qabs [H, M, R] -> out [M, H*(R+rd)]
 template <typename T>
 __global__ __launch_bounds__(256) void latent_q_pack_kernel(
-    const T* __restrict__ q, const T* __restrict__ qabs,
+    const T* __restrict__ q, const int64_t ld, const T* __restrict__ qabs,
     const float* __restrict__ freq, const int* __restrict__ pos,
     T* __restrict__ out, const int Tn, const int64_t M, const int H,
     const int d, const int np, const int R) {
@@ -77,7 +77,7 @@ __global__ __launch_bounds__(256) void latent_q_pack_kernel(
     sincosf(p * freq[i], &sn_s[i], &cs_s[i]);
   __syncthreads();
   const int rd = 2 * np, D = R + rd;
-  const T* qr = q + row * (int64_t)H * (d + rd);
+  const T* qr = q + row * ld;
   T* orow = out + row * (int64_t)H * D;
   for (int idx = threadIdx.x; idx < H * R; idx += blockDim.x) {
     const int h = idx / R, i = idx % R;
@@ -148,8 +148,9 @@ void latent_q_pack(torch::Tensor q, torch::Tensor qabs, torch::Tensor rot_freq,
   DNET_CHECK(T > 0 && M % T == 0, "rows = B*T");
   const int64_t np = rot_freq.numel();
   DNET_CHECK(np <= kMaxPairs, "rotated size <= 256");
+  // columns after the queries (the rest of a fused projection) are ignored
   DNET_CHECK(q.dim() == 2 && q.is_contiguous() &&
-                 q.size(1) == H * (d + 2 * np), "q [B*T, H*(d+rd)]");
+                 q.size(1) >= H * (d + 2 * np), "q [B*T, >= H*(d+rd)]");
   DNET_CHECK(qabs.dim() == 3 && qabs.is_contiguous() && qabs.size(0) == H &&
                  qabs.size(1) == M && qabs.scalar_type() == q.scalar_type(),
              "qabs [H, B*T, R]");
@@ -165,7 +166,7 @@ void latent_q_pack(torch::Tensor q, torch::Tensor qabs, torch::Tensor rot_freq,
   auto st = current_stream();
 #define LQ(TT)                                                               \
   hipLaunchKernelGGL((latent_q_pack_kernel<TT>), dim3((unsigned)M),          \
-                     dim3(256), 0, st, (const TT*)q.data_ptr(),              \
+                     dim3(256), 0, st, (const TT*)q.data_ptr(), q.size(1),   \
                      (const TT*)qabs.data_ptr(),                             \
                      rot_freq.data_ptr<float>(), pos.data_ptr<int>(),        \
                      (TT*)out.data_ptr(), (int)T, M, (int)H, (int)d,         \

@@ -1361,6 +1361,13 @@ def moe_plan(idx: torch.Tensor, E: int):
             torch.bincount(flat, minlength=E).to(torch.int32))
 
 
+def moe_gather(x: torch.Tensor, order: torch.Tensor, val: torch.Tensor):
+    """Rows and scales of sorted entries (``moe_plan``): entry t*top + k is
+    row t of x [T, W] with scale val[t, k]."""
+    entry = order.long()
+    return x[entry // val.shape[1]], val.reshape(-1)[entry]
+
+
 def moe_gateup_rows(x: torch.Tensor, w: torch.Tensor,
                     we: torch.Tensor) -> torch.Tensor:
     """Experts' first half on every row, inputs scaled by the routing

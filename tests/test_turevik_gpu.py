@@ -1,0 +1,332 @@
+"""GPU numerics of the Turevik kernels (norm with token shift, minGRU
+recurrence, raw cache append, gated activations, sigmoid router with plan /
+gather / merge, the experts' row kernels, sinks on shared latent rows) against
+their plain-PyTorch references (dnet_amd.ops.reference), in bf16 and fp32,
+with ragged batches, slot indirection, continued states and sizes that are not
+multiples of the kernels' tiles; and the whole model on the GPU (prefill,
+graph-captured decode) against the same model on the CPU."""
+import pytest
+import torch
+
+import dnet_amd.ops as ops
+from dnet_amd.ops import reference as ref
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda:0"
+DTS = [torch.bfloat16, torch.float32]
+
+
+def _tol(dt):
+    return dict(atol=3e-2, rtol=3e-2) if dt == torch.bfloat16 \
+        else dict(atol=3e-5, rtol=3e-5)
+
+
+def _i32(v):
+    return torch.tensor(v, dtype=torch.int32)
+
+
+def _geo(T):
+    """Three rows of a ragged batch: continued, fresh and short, padding."""
+    return _i32([40, 0, 7]), _i32([T, min(2, T), 0]), _i32([3, 0, 1])
+
+
+@pytest.mark.parametrize("odt", DTS)
+@pytest.mark.parametrize("W,T", [(64, 37), (36, 5), (1030, 19), (7, 3),
+                                 (4096, 70), (50, 2)])
+def test_norm_token_shift(odt, W, T):
+    torch.manual_seed(W + T)
+    B, Bc = 3, 4
+    x = torch.randn(B * T, W, device=DEV) * 2
+    wn = 1 + 0.2 * torch.randn(W, device=DEV)
+    wa = 1 + 0.2 * torch.randn(W, device=DEV)
+    mu = torch.rand(W, device=DEV)
+    a = torch.randn(B * T, W, device=DEV).to(odt)
+    pos, lens, slots = _geo(T)
+    prev = torch.randn(Bc, W, device=DEV)
+    for fused in (False, True):
+        pg, pr = prev.clone(), prev.cpu().clone()
+        xg, xr = x.clone(), x.cpu().clone()
+        args = (pos, T, 1e-6, odt, lens, slots)
+        gargs = (pos.to(DEV), T, 1e-6, odt, lens.to(DEV), slots.to(DEV))
+        if fused:
+            y = ops.resid_norm_token_shift(xg, a, wa, wn, mu, pg, *gargs)
+            want = ref.resid_norm_token_shift(
+                xr, a.cpu(), wa.cpu(), wn.cpu(), mu.cpu(), pr, *args)
+        else:
+            y = ops.norm_token_shift(xg, wn, mu, pg, *gargs)
+            want = ref.norm_token_shift(xr, wn.cpu(), mu.cpu(), pr, *args)
+        for b in range(B):
+            s = slice(b * T, b * T + int(lens[b]))
+            torch.testing.assert_close(y[s].cpu().float(), want[s].float(),
+                                       **_tol(odt))
+        assert torch.isfinite(y.float()).all()
+        torch.testing.assert_close(pg.cpu(), pr, atol=3e-5, rtol=3e-5)
+        torch.testing.assert_close(xg.cpu(), xr, atol=3e-5, rtol=3e-5)
+        # decode steps go on from the state the portion left; row 2 is idle
+        for step in range(3):
+            x1 = torch.randn(B, W, device=DEV)
+            a1 = torch.randn(B, W, device=DEV).to(odt)
+            x1r = x1.cpu().clone()
+            p1 = (pos + lens + step).to(torch.int32)
+            idle = _i32([1, 1, 0])
+            y = ops.resid_norm_token_shift(
+                x1, a1, wa, wn, mu, pg, p1.to(DEV), 1, 1e-6, odt,
+                idle.to(DEV), slots.to(DEV))
+            want = ref.resid_norm_token_shift(
+                x1r, a1.cpu(), wa.cpu(), wn.cpu(), mu.cpu(), pr, p1, 1, 1e-6,
+                odt, idle, slots)
+            torch.testing.assert_close(y[:2].cpu().float(), want[:2].float(),
+                                       **_tol(odt))
+            torch.testing.assert_close(x1.cpu(), x1r, atol=3e-5, rtol=3e-5)
+        torch.testing.assert_close(pg.cpu(), pr, atol=3e-5, rtol=3e-5)
+
+
+@pytest.mark.parametrize("dt", DTS)
+@pytest.mark.parametrize("N,T", [(64, 37), (36, 300), (1030, 19), (7, 3),
+                                 (130, 64), (65, 65), (200, 513)])
+def test_mingru_scan(dt, N, T):
+    torch.manual_seed(N + T)
+    B, Bc = 3, 4
+    ld = 3 * N + 11
+    z0, x0, g0 = 3, 3 + N, 6 + 2 * N
+    src = torch.randn(B * T, ld, device=DEV).to(dt)
+    bz, bx = torch.randn(N, device=DEV) - 1, torch.randn(N, device=DEV)
+    bz[0] = -30.0                        # a channel that keeps its state
+    pos, lens, slots = _geo(T)
+    st = torch.randn(Bc, N, device=DEV)
+    sr = st.cpu().clone()
+
+    def both(src, pos, T, lens):
+        y = ops.mingru_scan(src, z0, x0, g0, bz, bx, st, pos.to(DEV), T,
+                            lens.to(DEV), slots.to(DEV))
+        want = ref.mingru_scan(src.cpu(), z0, x0, g0, bz.cpu(), bx.cpu(), sr,
+                               pos, T, lens, slots)
+        torch.testing.assert_close(y.cpu().float(), want.float(), **_tol(dt))
+        torch.testing.assert_close(st.cpu(), sr, atol=5e-5, rtol=5e-5)
+
+    both(src, pos, T, lens)
+    for step in range(3):
+        both(torch.randn(B, ld, device=DEV).to(dt),
+             (pos + lens + step).to(torch.int32), 1, _i32([1, 1, 0]))
+
+
+@pytest.mark.parametrize("sdt,cdt", [(torch.bfloat16, torch.bfloat16),
+                                     (torch.float32, torch.bfloat16),
+                                     (torch.float32, torch.float32)])
+def test_cache_append(sdt, cdt):
+    torch.manual_seed(3)
+    B, T, Bc, H, D, S = 3, 9, 4, 3, 20, 64
+    src = torch.randn(B * T, 5 + H * D + 2, device=DEV).to(sdt)
+    cache = torch.randn(Bc, H, S, D, device=DEV).to(cdt)
+    cr = cache.cpu().clone()
+    pos, lens, slots = _geo(T)
+    ops.cache_append(src, 5, cache, pos.to(DEV), T, lens.to(DEV),
+                     slots.to(DEV))
+    ref.cache_append(src.cpu(), 5, cr, pos, T, lens, slots)
+    assert torch.equal(cache.cpu(), cr)
+
+
+@pytest.mark.parametrize("dt", DTS)
+@pytest.mark.parametrize("act", ["silu", "gelu_tanh"])
+@pytest.mark.parametrize("I", [64, 36, 1030, 7])
+def test_gated_act(dt, act, I):
+    torch.manual_seed(I)
+    gu = (torch.randn(9, 2 * I, device=DEV) * 2).to(dt)
+    gu[0, 0], gu[1, 0] = 60.0, -60.0     # saturated gates
+    for scale in (None, torch.rand(9, device=DEV)):
+        y = ops.gated_act(gu, act, scale)
+        want = ref.gated_act(gu.cpu(), act,
+                             None if scale is None else scale.cpu())
+        torch.testing.assert_close(y.cpu().float(), want.float(), **_tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTS)
+@pytest.mark.parametrize("T,W,E,top,sg", [(1, 64, 5, 1, True),
+                                          (40, 50, 12, 3, False),
+                                          (33, 256, 70, 8, True),
+                                          (300, 128, 9, 2, True),
+                                          (257, 36, 130, 5, False),
+                                          (5, 32, 4, 4, True),
+                                          (6, 40, 1, 1, False)])
+def test_router_plan_gather_merge(dt, T, W, E, top, sg):
+    torch.manual_seed(T + E)
+    x = torch.randn(T, W, device=DEV).to(dt)
+    w = torch.randn(E + sg, W, device=DEV)
+    idx, val, we, gate = ops.moe_router(x, w, E, top)
+    ri, rv, rw, rg = ref.moe_router(x.cpu(), w.cpu(), E, top)
+    assert torch.equal(idx.cpu(), ri)
+    for a, b in ((val, rv), (we, rw)) + (((gate, rg),) if sg else ()):
+        torch.testing.assert_close(a.cpu(), b, atol=2e-5, rtol=2e-5)
+    assert sg or gate is None
+    order, at, counts = ops.moe_plan(idx, E)
+    ro, ra, rc = ref.moe_plan(ri, E)
+    assert torch.equal(order.cpu(), ro) and torch.equal(at.cpu(), ra) \
+        and torch.equal(counts.cpu(), rc)
+    xs, scale = ops.moe_gather(x, order, val)
+    rx, rs = ref.moe_gather(x.cpu(), ro, rv)
+    assert torch.equal(xs.cpu(), rx)
+    torch.testing.assert_close(scale.cpu(), rs, atol=2e-5, rtol=2e-5)
+    y = torch.randn(T * top, W, device=DEV).to(dt)
+    sh = torch.randn(T, W, device=DEV).to(dt) if sg else None
+    got = ops.moe_merge(y, at, sh, gate, dt)
+    want = ref.moe_merge(y.cpu(), ra, None if sh is None else sh.cpu(), rg,
+                         dt)
+    torch.testing.assert_close(got.cpu().float(), want.float(), **_tol(dt))
+    y = torch.randn(E, T, W, device=DEV).to(dt)
+    got = ops.moe_merge(y, idx, sh, gate, dt)
+    want = ref.moe_merge(y.cpu(), ri, None if sh is None else sh.cpu(), rg,
+                         dt)
+    torch.testing.assert_close(got.cpu().float(), want.float(), **_tol(dt))
+
+
+@pytest.mark.parametrize("T,W,I,E,top", [(1, 64, 32, 5, 1), (7, 72, 40, 6, 2),
+                                         (16, 320, 64, 12, 1),
+                                         (32, 1024, 512, 8, 2),
+                                         (33, 200, 24, 3, 3),
+                                         (64, 136, 104, 4, 1),
+                                         (100, 64, 48, 5, 2)])
+def test_expert_row_kernels(T, W, I, E, top):
+    """All row-block sizes, inner sizes off the 32-wide step, column tails,
+    experts that nobody chose."""
+    torch.manual_seed(T + W)
+    dt = torch.bfloat16
+    x = torch.randn(T, W, device=DEV).to(dt)
+    w1 = (torch.randn(E, 2 * I, W, device=DEV) * W ** -0.5).to(dt)
+    w2 = (torch.randn(E, W, I, device=DEV) * I ** -0.5).to(dt)
+    router = torch.randn(E, W, device=DEV) * W ** -0.5
+    if E > top:
+        router[0] = 0.0
+        router[0, 0] = -100.0            # nobody takes expert 0 ...
+        x[:, 0] = 3.0
+    idx, val, we, _ = ops.moe_router(x, router, E, top)
+    if E > top:
+        assert not bool((idx == 0).any())
+    act = ops.moe_gateup_rows(x, w1, we)
+    want = ref.moe_gateup_rows(x.cpu(), w1.cpu(), we.cpu())
+    y = ops.moe_down_rows(act, w2, we)
+    wy = ref.moe_down_rows(act.cpu(), w2.cpu(), we.cpu())
+    for e in range(E):
+        rows = (idx == e).any(dim=1).cpu()
+        torch.testing.assert_close(act[e].cpu().float()[rows],
+                                   want[e].float()[rows], **_tol(dt))
+        torch.testing.assert_close(y[e].cpu().float()[rows],
+                                   wy[e].float()[rows], **_tol(dt))
+    out = ops.moe_merge(y, idx, None, None, dt)
+    full = sum(ref.moe_down_rows(want, w2.cpu(), we.cpu()).float()
+               * (we.cpu().t() > 0).unsqueeze(-1))
+    torch.testing.assert_close(out.cpu().float(), full, **_tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTS)
+@pytest.mark.parametrize("H,R,rd", [(4, 96, 32), (3, 20, 6), (16, 64, 32),
+                                    (32, 192, 64)])
+def test_sink_on_shared_rows(dt, H, R, rd):
+    """Attention against shared latent rows with a sink that matters, in
+    prompts and in decoding (rows, prompt and grouped-heads kernels)."""
+    torch.manual_seed(H + R)
+    B, T, Bc, S = 3, 45, 4, 192
+    D = R + rd
+    rows = torch.randn(Bc, 1, S, D, device=DEV).to(dt)
+    sinks = torch.randn(H, device=DEV) + 3.0
+    for Tq in (T, 1):
+        pos, lens, slots = _geo(Tq)
+        pos = _i32([100, 0, 7])
+        q = torch.randn(B * Tq, H * D, device=DEV).to(dt)
+        out = ops.attn_mod(q, rows, None, pos.to(DEV), Tq, D ** -0.5,
+                           lens.to(DEV), slots.to(DEV), sinks=sinks, v_dim=R)
+        want = ref.attn_mod(q.cpu(), rows.cpu(), None, pos, Tq, D ** -0.5,
+                            lens, slots, sinks=sinks.cpu(), v_dim=R)
+        other = ref.attn_mod(q.cpu(), rows.cpu(), None, pos, Tq, D ** -0.5,
+                             lens, slots, v_dim=R)
+        for b in range(B):
+            s = slice(b * Tq, b * Tq + int(lens[b]))
+            torch.testing.assert_close(out[s].cpu().float(),
+                                       want[s].float(), **_tol(dt))
+        assert float((other - want).abs().max()) > 0.3
+
+
+def _executors(dtype, kw, mb=4, smax=256, width=96, vocab=200):
+    from dnet_amd.models import ModelConfig
+    from dnet_amd.models.config import turevik_config
+    from dnet_amd.parallel.ring import RingExecutor
+    from turevik_oracle import make_checkpoint
+    # bfloat16: the two paths round differently and every layer of a random
+    # stack multiplies that noise, so the bfloat16 stack is shallow
+    hf = turevik_config(width, vocab, "lsgs",
+                        layers=6 if dtype == "float32" else 3, **kw)
+    sd = make_checkpoint(hf, seed=11,
+                         out_gain=1.0 if dtype == "float32" else 0.5)
+    out = []
+    for dev, graphs in (("cpu", False), (DEV, True)):
+        cfg = ModelConfig.from_hf(hf)
+        cfg.compute_dtype = dtype
+        ex = RingExecutor(cfg, 0, 1, torch.device(dev), mb_size=mb,
+                          smax=smax, use_graphs=graphs, init_weights=False)
+        ex.model.load_state_dict(sd)
+        out.append(ex)
+    return out
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("kw", [
+    {}, dict(shared_ff=0, top=1, experts=7, gru_width=40),
+    dict(heads=3, dim=10, rot_dim=6, vdim=12, kv_rank=20, experts=0, ff=100),
+    dict(heads=16, dim=16, rot_dim=8, vdim=24, kv_rank=40, top=4)])
+def test_model_gpu_equals_cpu(dtype, kw):
+    """Ragged prompt batch into scattered slots (rows enough for the sorted
+    expert path), a second portion, then graph-captured decode steps with an
+    idle row: the GPU kernels against the CPU reference ops under the same
+    executor."""
+    torch.manual_seed(0)
+    prompts = [torch.randint(0, 200, (n,)) for n in (41, 3, 17)]
+    more = [torch.randint(0, 200, (n,)) for n in (2, 9, 1)]
+    steps = [torch.randint(0, 200, (4,)) for _ in range(5)]
+    outs = []
+    for ex in _executors(dtype, kw):
+        rows = [r.float().cpu() for r in ex.prefill_slots(
+            [2, 0, 3], prompts, want=[list(range(41)), [2], [0, 16]])]
+        rows += [r.float().cpu() for r in ex.prefill_slots(
+            [2, 0, 3], more, want=[[0, 1], [8], [0]], start=[41, 3, 17])]
+        for i, t in enumerate(steps):
+            ex.tokbuf[0].copy_(t)
+            idle = torch.tensor([False, True, False, i % 2 == 1])
+            ex.slot_step_compute(park=idle.to(ex.device))
+            live = [j for j in range(4) if not bool(idle[j]) and j != 1]
+            rows.append(ex.logits_buf[0].float().cpu()[live].clone())
+            ex.kvs[0].pos.add_((~idle).to(torch.int32).to(ex.device))
+        if ex.device.type == "cuda":
+            assert ex.use_graphs and ex._graphs     # captured, not eager
+        outs.append(torch.cat(rows))
+    cpu, gpu = outs
+    err = (gpu - cpu).pow(2).mean(-1).sqrt() / cpu.pow(2).mean().sqrt()
+    if dtype == "float32":
+        assert float(err.max()) < 1e-3, err
+    else:
+        # a close routing call may fall the other way in single rows
+        assert float(err.median()) < 0.05, err
+        assert float((err > 0.2).float().mean()) < 0.1, err
+
+
+@pytest.mark.parametrize("dtype", ["bfloat16", "float32"])
+def test_odd_sizes_gpu_matches_cpu(dtype):
+    """Sizes that are multiples of nothing: every kernel's unvectorized path
+    and the fallbacks of the linears and of the experts."""
+    kw = dict(heads=3, dim=7, rot_dim=2, vdim=5, kv_rank=21, gru_width=37,
+              ff=37, experts=5, top=2, expert_ff=13, shared_ff=11)
+    prompts = [torch.arange(19) % 77, (torch.arange(3) * 7) % 77]
+    outs = []
+    for ex in _executors(dtype, kw, mb=2, smax=64, width=50, vocab=77):
+        rows = [r.float().cpu() for r in ex.prefill_slots(
+            [1, 0], prompts, want=[list(range(19)), [2]])]
+        for step in range(3):
+            ex.tokbuf[0].copy_(torch.tensor([5 + step, 9 + step]))
+            ex.slot_step_compute(park=torch.zeros(2, dtype=torch.bool,
+                                                  device=ex.device))
+            rows.append(ex.logits_buf[0].float().cpu().clone())
+            ex.kvs[0].pos.add_(1)
+        outs.append(torch.cat(rows))
+    cpu, gpu = outs
+    err = (gpu - cpu).pow(2).mean(-1).sqrt() / cpu.pow(2).mean().sqrt()
+    assert float(err.median()) < (2e-4 if dtype == "float32" else 0.05)
+    assert float((err > (1e-3 if dtype == "float32" else 0.2)).float()
+                 .mean()) < 0.1, err
