@@ -964,7 +964,7 @@ def moe_router(x, w, E: int, top: int):
         if T <= _ROUTER_FUSED_ROWS:
             _native().moe_router(x, w, None, idx, val, we, gate)
         else:
-            _native().moe_router(None, None, x.float() @ w.t(), idx, val, we,
+            _native().moe_router(None, w, x.float() @ w.t(), idx, val, we,
                                  gate)
         return idx, val, we, gate
     return ref.moe_router(x, w, E, top)

@@ -37,8 +37,9 @@ bool is_i32(const torch::Tensor& t) { return t.scalar_type() == torch::kInt32; }
 // ---- router ------------------------------------------------------------------
 // One workgroup per row. x given: 256 threads form the R = E (+1) dot products
 // (wave per router row); else one wave starts from logits [T, R]. Then the
-// first wave picks: scores sit in LDS, every lane scans its experts, ties go
-// to the lower expert.
+// first wave picks by the logits (the sigmoid keeps their order, and does not
+// tell large ones apart in fp32): they sit in LDS, every lane scans its
+// experts, ties go to the lower expert.
 template <typename T>
 __global__ __launch_bounds__(256) void moe_router_kernel(
     const T* __restrict__ x, const float* __restrict__ w,
@@ -75,17 +76,16 @@ __global__ __launch_bounds__(256) void moe_router_kernel(
   }
   __syncthreads();
   for (int e = threadIdx.x; e < R; e += blockDim.x) {
-    float s = 1.f / (1.f + expf(-sc[e]));
-    if (!(s == s)) s = 0.f;                 // padding rows may hold anything
-    sc[e] = s;
-    if (e == E && gate) gate[t] = s;
+    const float z = sc[e];
+    sc[e] = z > -1e30f ? z : -1e30f;        // (padding rows may hold NaN)
+    if (e == E && gate) gate[t] = 1.f / (1.f + expf(-z));
     if (e < E) we[(int64_t)t * E + e] = 0.f;
   }
   __syncthreads();
   if (wid != 0) return;
   for (int k = 0; k < top; ++k) {
-    float bv = -1.f;
-    int bi = E;                             // chosen scores are set to -1
+    float bv = -2e38f;
+    int bi = E;                             // chosen logits are set to -3e38
     for (int e = lane; e < E; e += 64) {
       const float s = sc[e];
       if (s > bv) {
@@ -102,13 +102,14 @@ __global__ __launch_bounds__(256) void moe_router_kernel(
         bi = oi;
       }
     }
-    // top <= E and scores >= 0: bi is always one of the experts
+    // top <= E: bi is always one of the experts
     if (lane == 0) {
+      const float s = 1.f / (1.f + expf(-bv));
       idx[(int64_t)t * top + k] = bi;
-      val[(int64_t)t * top + k] = bv;
+      val[(int64_t)t * top + k] = s;
       // never 0: a chosen expert must not look skipped to the row kernels
-      we[(int64_t)t * E + bi] = fmaxf(bv, 1e-38f);
-      sc[bi] = -1.f;
+      we[(int64_t)t * E + bi] = fmaxf(s, 1e-38f);
+      sc[bi] = -3e38f;
     }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // one wave only
   }

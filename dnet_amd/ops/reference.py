@@ -1323,11 +1323,13 @@ def moe_router(x: torch.Tensor, w: torch.Tensor, E: int, top: int):
     """Sigmoid router in fp32. x [T, W], w fp32 [E or E+1, W] (the last row,
     when there, is the shared expert's gate). Returns (idx int32 [T, top],
     val fp32 [T, top], we fp32 [T, E] with the values of the chosen experts
-    and 0 elsewhere, gate fp32 [T] or None)."""
-    z = torch.sigmoid(x.float() @ w.t())
+    and 0 elsewhere, gate fp32 [T] or None). The choice is made on the logits
+    (the sigmoid keeps their order, and rounds large ones to equal)."""
+    z = x.float() @ w.t()
     val, idx = torch.topk(z[:, :E], top, dim=-1)
+    val = torch.sigmoid(val)
     we = torch.zeros_like(z[:, :E]).scatter_(1, idx, val)
-    gate = z[:, E].contiguous() if w.shape[0] > E else None
+    gate = torch.sigmoid(z[:, E]) if w.shape[0] > E else None
     return idx.to(torch.int32), val, we, gate
 
 

@@ -151,7 +151,7 @@ def test_gated_act(dt, act, I):
 def test_router_plan_gather_merge(dt, T, W, E, top, sg):
     torch.manual_seed(T + E)
     x = torch.randn(T, W, device=DEV).to(dt)
-    w = torch.randn(E + sg, W, device=DEV)
+    w = torch.randn(E + sg, W, device=DEV) * 2 * W ** -0.5
     idx, val, we, gate = ops.moe_router(x, w, E, top)
     ri, rv, rw, rg = ref.moe_router(x.cpu(), w.cpu(), E, top)
     assert torch.equal(idx.cpu(), ri)
