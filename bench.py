@@ -56,7 +56,19 @@ _COMPARE_SIZES = [("2k", 2048, 16, 4, 128, 8192),
 def _family_hf(fam, W, H, KV, D, FF, layers, vocab, args):
     """config.json-style description of ``fam`` at the given layer sizes."""
     from dnet_amd.models.config import (gegorax_config, komizen_config,
-                                        lurisun_config, posudra_config)
+                                        lurisun_config, posudra_config,
+                                        turevik_config)
+    if fam == "turevik":
+        # layers of four kinds in turn: latent attention with rows of its
+        # own, two latent-attention layers on those rows, a minGRU over the
+        # model width between them; 192 + 64 cached entries per token and
+        # row-owning layer; a dense feed-forward in layer 0, then mixtures
+        # of gated experts (2 chosen of 8) with a shared expert
+        E = args.compare_experts or 8
+        return turevik_config(
+            W, vocab, "lsgs", layers=layers, heads=H, dim=D, rot_dim=64,
+            vdim=D, kv_rank=192, ff=FF, experts=E, top=min(2, E),
+            expert_ff=FF // 4, shared_ff=FF // 4)
     if fam == "lurisun":
         # constant-decay linear attention, windowed latent attention and
         # chunked sigmoid attention in turn; linear-attention heads of D x D
@@ -112,7 +124,8 @@ def _family_hf(fam, W, H, KV, D, FF, layers, vocab, args):
 
 # family -> the closest existing family it is measured beside
 _COMPARE_WITH = {"posudra": "qwen3", "gegorax": "posudra",
-                 "komizen": "gegorax", "lurisun": "gegorax"}
+                 "komizen": "gegorax", "lurisun": "gegorax",
+                 "turevik": "komizen"}
 
 
 def compare_family(args, device):
@@ -122,8 +135,9 @@ def compare_family(args, device):
     komizen: gegorax — attention beside state-space and delta-rule layers on
     an fp32 residual with per-slot recurrent state; lurisun: gegorax —
     windowed attention beside linear recurrences with per-slot state, dense
-    feed-forwards, fp32 residual) at
-    equal layer sizes, bf16, random weights. One JSON line; the default
+    feed-forwards, fp32 residual; turevik: komizen — latent attention on
+    shared rows, recurrent layers with per-slot state, mixtures of experts)
+    at equal layer sizes, bf16, random weights. One JSON line; the default
     workload is untouched."""
     new, old = args.compare_family, _COMPARE_WITH[args.compare_family]
     layers, vocab = args.compare_layers, 32768
@@ -211,7 +225,8 @@ def main():
                     help="GPU-resident layers per rank (0=all; <local layers "
                          "enables host-DRAM weight streaming)")
     ap.add_argument("--compare-family", default="",
-                    choices=["", "posudra", "gegorax", "komizen", "lurisun"],
+                    choices=["", "posudra", "gegorax", "komizen", "lurisun",
+                             "turevik"],
                     help="instead of the default workload: throughput of "
                          "this family beside its closest existing one at "
                          "equal layer sizes")
@@ -219,7 +234,7 @@ def main():
     ap.add_argument("--compare-experts", type=int, default=0,
                     help="gegorax: experts of the mixture feed-forward in "
                          "every second layer (0 = dense feed-forwards); "
-                         "komizen: experts of every layer (0 = 8)")
+                         "komizen, turevik: experts of every mixture (0 = 8)")
     ap.add_argument("--compare-prefill-batch", type=int, default=8)
     ap.add_argument("--compare-sizes", default="",
                     help="comma list out of 2k,4k,5k (default: all)")

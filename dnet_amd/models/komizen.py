@@ -491,13 +491,17 @@ class KomizenRingModel(RingModel):
             return ops.moe_down(act, lw.down_w, None, None, we, 0, False)
         if T <= self.DENSE_MOE_MAX_T:
             # a decode batch that reaches most experts anyway: every expert
-            # on every row as two batched products (each expert's weights
-            # read once), weighted with zero for the experts a row did not
-            # choose; no host sync
-            z = torch.bmm(u.unsqueeze(0).expand(E, T, W),
-                          lw.up_w.transpose(1, 2))              # [E, T, I]
-            a = ops.act_slice(z.view(E * T, I), 0, I, "relu_sq")
-            d = torch.bmm(a.view(E, T, I), lw.down_w.transpose(1, 2))
+            # on every row (each expert's weights read once), weighted with
+            # zero for the experts a row did not choose; no host sync
+            if self.wdtype == torch.bfloat16 and W % 8 == 0 and I % 8 == 0:
+                act = ops.moe_up_rows(u, lw.up_w, we)
+                d = ops.moe_down_rows(act, lw.down_w, we)
+            else:
+                z = torch.bmm(u.unsqueeze(0).expand(E, T, W),
+                              lw.up_w.transpose(1, 2).contiguous())
+                a = ops.act_slice(z.view(E * T, I), 0, I, "relu_sq")
+                d = torch.bmm(a.view(E, T, I),
+                              lw.down_w.transpose(1, 2).contiguous())
             return ops.moe_weighted_sum(d, we)
         out = torch.zeros(T, W, dtype=torch.float32, device=u.device)
         hit = (we > 0).any(dim=0).tolist()

@@ -1008,6 +1008,18 @@ def moe_gateup_rows(x, w, we) -> torch.Tensor:
     return ref.moe_gateup_rows(x, w, we)
 
 
+def moe_up_rows(x, w, we) -> torch.Tensor:
+    """``moe_up_act`` on the matrix cores, for decode-sized batches that
+    reach most experts: act [E, T, I] = relu(x w_e^T)^2 in bf16, experts no
+    row chose unwritten."""
+    if x.is_cuda:
+        act = torch.empty(w.shape[0], x.shape[0], w.shape[1], dtype=x.dtype,
+                          device=x.device)
+        _native().moe_up_rows(x, w, we, act)
+        return act
+    return ref.moe_up_act(x, w, we)
+
+
 def moe_down_rows(act, w, we) -> torch.Tensor:
     """Second half of ``moe_gateup_rows``: [E, T, N], skipped experts
     unwritten; ``moe_merge`` reads the chosen ones only."""

@@ -209,6 +209,8 @@ void moe_gather(torch::Tensor x, torch::Tensor order, torch::Tensor val,
                 torch::Tensor xs, torch::Tensor scale);
 void moe_gateup_rows(torch::Tensor x, torch::Tensor w, torch::Tensor we,
                      torch::Tensor act);
+void moe_up_rows(torch::Tensor x, torch::Tensor w, torch::Tensor we,
+                 torch::Tensor act);
 void moe_down_rows(torch::Tensor act, torch::Tensor w, torch::Tensor we,
                    torch::Tensor y);
 void moe_merge(torch::Tensor y, torch::Tensor at,
@@ -334,6 +336,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("moe_gather", &dnet::moe_gather, "rows and scales of sorted entries");
   m.def("moe_gateup_rows", &dnet::moe_gateup_rows,
         "gated experts on a decode batch, inputs scaled (matrix cores)");
+  m.def("moe_up_rows", &dnet::moe_up_rows,
+        "ungated experts (squared ReLU) on a decode batch (matrix cores)");
   m.def("moe_down_rows", &dnet::moe_down_rows,
         "experts' down projection on a decode batch (matrix cores)");
   m.def("moe_merge", &dnet::moe_merge,

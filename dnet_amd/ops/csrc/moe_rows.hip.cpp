@@ -7,11 +7,11 @@
 //   moe_plan         entries (row, choice) sorted by expert, without host work
 //   moe_gather       the sorted entries' rows and scales
 //   moe_gateup_rows  every expert on every row of a decode batch, matrix
-//   moe_down_rows    cores: an expert's weights are read once for all rows,
+//   moe_down_rows    cores (moe_up_rows: ungated experts, squared ReLU): an expert's weights are read once for all rows,
 //                    experts that no row chose are skipped on the device
 //   moe_merge        sum of each row's chosen results + gate * shared
 //
-// The scale w of an input commutes with the product, so it is applied to the
+// The scale w of a gated expert's input commutes with the product, so it is applied to the
 // fp32 accumulators: silu(w g) * (w u). A row that did not choose an expert
 // has w = 0 and therefore act = 0. "short" stands for bf16 bits.
 #include "common.h"
@@ -35,13 +35,23 @@ bool is_f32(const torch::Tensor& t) { return t.scalar_type() == torch::kFloat32;
 bool is_i32(const torch::Tensor& t) { return t.scalar_type() == torch::kInt32; }
 
 // ---- router ------------------------------------------------------------------
-// One workgroup per row. x given: 256 threads form the R = E (+1) dot products
-// (wave per router row); else one wave starts from logits [T, R]. Then the
+// One workgroup per row. x given: its waves form the R = E (+1) dot products
+// (wave per router row, up to 16 waves); else one wave starts from logits [T, R]. Then the
 // first wave picks by the logits (the sigmoid keeps their order, and does not
 // tell large ones apart in fp32): they sit in LDS, every lane scans its
 // experts, ties go to the lower expert.
+template <typename T> __device__ __forceinline__ float4 ld4(const T* p);
+template <> __device__ __forceinline__ float4 ld4<float>(const float* p) {
+  return *reinterpret_cast<const float4*>(p);
+}
+template <> __device__ __forceinline__ float4 ld4<short>(const short* p) {
+  const short4v v = *reinterpret_cast<const short4v*>(p);
+  return make_float4(bits2f(v.x[0]), bits2f(v.x[1]), bits2f(v.x[2]),
+                     bits2f(v.x[3]));
+}
+
 template <typename T>
-__global__ __launch_bounds__(256) void moe_router_kernel(
+__global__ __launch_bounds__(1024) void moe_router_kernel(
     const T* __restrict__ x, const float* __restrict__ w,
     const float* __restrict__ logits, int* __restrict__ idx,
     float* __restrict__ val, float* __restrict__ we, float* __restrict__ gate,
@@ -57,13 +67,33 @@ __global__ __launch_bounds__(256) void moe_router_kernel(
       const float* wr = w + (int64_t)e * W;
       float s = 0.f;
       if ((W & 3) == 0) {
-        for (int i = lane * 4; i < W; i += 256) {
-          const float4 wv = *reinterpret_cast<const float4*>(wr + i);
-          s = fmaf(ldx<T>(xr + i), wv.x, s);
-          s = fmaf(ldx<T>(xr + i + 1), wv.y, s);
-          s = fmaf(ldx<T>(xr + i + 2), wv.z, s);
-          s = fmaf(ldx<T>(xr + i + 3), wv.w, s);
+        // 4 pieces in flight
+        float4 a = {0.f, 0.f, 0.f, 0.f};
+        int i = lane * 4;
+        for (; i + 768 < W; i += 1024) {
+          float4 wv[4], xv[4];
+#pragma unroll
+          for (int u = 0; u < 4; ++u) {
+            wv[u] = *reinterpret_cast<const float4*>(wr + i + u * 256);
+            xv[u] = ld4<T>(xr + i + u * 256);
+          }
+#pragma unroll
+          for (int u = 0; u < 4; ++u) {
+            a.x = fmaf(xv[u].x, wv[u].x, a.x);
+            a.y = fmaf(xv[u].y, wv[u].y, a.y);
+            a.z = fmaf(xv[u].z, wv[u].z, a.z);
+            a.w = fmaf(xv[u].w, wv[u].w, a.w);
+          }
         }
+        for (; i < W; i += 256) {
+          const float4 wv = *reinterpret_cast<const float4*>(wr + i);
+          const float4 xv = ld4<T>(xr + i);
+          a.x = fmaf(xv.x, wv.x, a.x);
+          a.y = fmaf(xv.y, wv.y, a.y);
+          a.z = fmaf(xv.z, wv.z, a.z);
+          a.w = fmaf(xv.w, wv.w, a.w);
+        }
+        s = (a.x + a.y) + (a.z + a.w);
       } else {
         for (int i = lane; i < W; i += 64) s = fmaf(ldx<T>(xr + i), wr[i], s);
       }
@@ -192,34 +222,39 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(
 }
 
 // ---- experts on the rows of a decode batch ----------------------------------------
-// grid (column tiles, row blocks of 16 MT, E), 4 waves. A wave owns every
-// fourth 32-wide step of the inner dimension (the four waves read neighbouring
-// pieces of the same weight rows), 4 weight fragments x MT row fragments of
-// v_mfma_f32_16x16x32_bf16; the partial sums meet in LDS. GLU: fragments
-// 0, 1 = gate columns, 2, 3 = the up columns beside them (32 columns of act);
-// else 64 columns.
-template <int MT, bool GLU>
-__global__ __launch_bounds__(256) void moe_rows_kernel(
+// grid (column tiles, row blocks of 16 MT, E), NW waves. A wave owns every
+// NW-th 32-wide step of the inner dimension (the waves read neighbouring
+// pieces of the same weight rows), NF weight fragments x MT row fragments of
+// v_mfma_f32_16x16x32_bf16, U steps in flight; the partial sums fold wave by
+// wave through LDS. GLU: the first half of the fragments are gate columns,
+// the second half the up columns beside them (8 NF columns of act), inputs
+// scaled by the routing weight; else 16 NF plain or squared-ReLU columns.
+constexpr int kPlain = 0, kGlu = 1, kReluSq = 2;
+
+template <int MT, int NF, int NW, int U, int KIND>
+__global__ __launch_bounds__(NW * 64) void moe_rows_kernel(
     const short* __restrict__ x, const short* __restrict__ w,
     const float* __restrict__ we, short* __restrict__ out, const int K,
     const int N, const int E, const int T, const int64_t x_expert) {
-  __shared__ f32x4 part[4][MT * 4][64];
+  constexpr bool GLU = KIND == kGlu;
+  constexpr int NC = GLU ? NF / 2 : NF;      // column fragments of the result
+  __shared__ f32x4 part[NW / 2][MT * NF][64];
   const int e = blockIdx.z;
   const int m0 = blockIdx.y * (16 * MT);
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   {
     const int t = m0 + lane;
     const bool hit = lane < 16 * MT && t < T && we[(int64_t)t * E + e] != 0.f;
-    if (__ballot(hit) == 0ull) return;       // the same in all four waves
+    if (__ballot(hit) == 0ull) return;       // the same in all waves
   }
   const int c = lane & 15, hi = lane >> 4;
-  const int n0 = blockIdx.x * (GLU ? 32 : 64);
-  const short* wp[4];
+  const int n0 = blockIdx.x * (16 * NC);
+  const short* wp[NF];
 #pragma unroll
-  for (int f = 0; f < 4; ++f) {
+  for (int f = 0; f < NF; ++f) {
     // GLU: w is [E, 2N, K] with the gate rows first
-    const int col = min(n0 + (GLU ? (f & 1) : f) * 16 + c, N - 1);
-    const int64_t row = GLU ? (int64_t)e * 2 * N + (f >> 1) * N + col
+    const int col = min(n0 + (f % NC) * 16 + c, N - 1);
+    const int64_t row = GLU ? ((int64_t)e * 2 + f / NC) * N + col
                             : (int64_t)e * N + col;
     wp[f] = w + row * K + hi * 8;
   }
@@ -227,105 +262,101 @@ __global__ __launch_bounds__(256) void moe_rows_kernel(
 #pragma unroll
   for (int m = 0; m < MT; ++m)
     xp[m] = x + e * x_expert + (int64_t)min(m0 + m * 16 + c, T - 1) * K + hi * 8;
-  f32x4 acc[MT][4];
+  f32x4 acc[MT][NF];
 #pragma unroll
   for (int m = 0; m < MT; ++m)
 #pragma unroll
-    for (int f = 0; f < 4; ++f) acc[m][f] = {0.f, 0.f, 0.f, 0.f};
+    for (int f = 0; f < NF; ++f) acc[m][f] = {0.f, 0.f, 0.f, 0.f};
 
-  // U steps of this wave in flight at a time
-  constexpr int U = MT >= 4 ? 2 : 4;
   const int full = K / 32;                   // whole steps
-  auto run = [&](const int s, auto cnt) {
+  // C steps s, s + NW, ... of this wave; `in`: the lane's 8 entries exist
+  auto run = [&](const int s, const bool in, auto cnt) {
     constexpr int C = decltype(cnt)::value;
-    bf16x8 wf[C][4], xf[C][MT];
+    bf16x8 wf[C][NF], xf[C][MT];
+    short8 z;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) z.x[j] = 0;
+    const bf16x8 zero = *reinterpret_cast<const bf16x8*>(&z);
 #pragma unroll
     for (int u = 0; u < C; ++u) {
+      const int at = (s + NW * u) * 32;
 #pragma unroll
-      for (int f = 0; f < 4; ++f)
-        wf[u][f] = *reinterpret_cast<const bf16x8*>(wp[f] + (s + 4 * u) * 32);
+      for (int f = 0; f < NF; ++f)
+        wf[u][f] = in ? *reinterpret_cast<const bf16x8*>(wp[f] + at) : zero;
 #pragma unroll
       for (int m = 0; m < MT; ++m)
-        xf[u][m] = *reinterpret_cast<const bf16x8*>(xp[m] + (s + 4 * u) * 32);
+        xf[u][m] = in ? *reinterpret_cast<const bf16x8*>(xp[m] + at) : zero;
     }
 #pragma unroll
     for (int u = 0; u < C; ++u)
 #pragma unroll
       for (int m = 0; m < MT; ++m)
 #pragma unroll
-        for (int f = 0; f < 4; ++f)
+        for (int f = 0; f < NF; ++f)
           acc[m][f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
               xf[u][m], wf[u][f], acc[m][f], 0, 0, 0);
   };
-  int s0 = wave;
-  for (; s0 + 4 * (U - 1) < full; s0 += 4 * U)
-    run(s0, std::integral_constant<int, U>{});
-  for (; s0 < full; s0 += 4) run(s0, std::integral_constant<int, 1>{});
-  if (full * 32 < K && wave == (full & 3)) { // the last, shorter step
-    const bool in = full * 32 + hi * 8 < K;  // K is a multiple of 8
-    short8 z;
-#pragma unroll
-    for (int j = 0; j < 8; ++j) z.x[j] = 0;
-    bf16x8 wf[4], xf[MT];
-#pragma unroll
-    for (int f = 0; f < 4; ++f)
-      wf[f] = in ? *reinterpret_cast<const bf16x8*>(wp[f] + full * 32)
-                 : *reinterpret_cast<const bf16x8*>(&z);
-#pragma unroll
-    for (int m = 0; m < MT; ++m)
-      xf[m] = in ? *reinterpret_cast<const bf16x8*>(xp[m] + full * 32)
-                 : *reinterpret_cast<const bf16x8*>(&z);
-#pragma unroll
-    for (int m = 0; m < MT; ++m)
-#pragma unroll
-      for (int f = 0; f < 4; ++f)
-        acc[m][f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xf[m], wf[f],
-                                                            acc[m][f], 0, 0, 0);
+  // every workgroup starts at another place of the inner dimension: weight
+  // rows are often a power of two apart, and workgroups in step would all
+  // read from the same few memory channels
+  const int groups = full / (NW * U);
+  const int turn =
+      groups > 1 ? (int)((blockIdx.x * 5 + blockIdx.z * 3) % groups) : 0;
+  for (int g = 0; g < groups; ++g) {
+    int gg = g + turn;
+    if (gg >= groups) gg -= groups;
+    run(gg * NW * U + wave, true, std::integral_constant<int, U>{});
   }
+  for (int s0 = groups * NW * U + wave; s0 < full; s0 += NW)
+    run(s0, true, std::integral_constant<int, 1>{});
+  if (full * 32 < K && wave == full % NW)    // the last, shorter step
+    run(full, full * 32 + hi * 8 < K,        // (K is a multiple of 8)
+        std::integral_constant<int, 1>{});
+
+#pragma unroll
+  for (int half = NW / 2; half > 0; half >>= 1) {
+    if (wave >= half && wave < 2 * half)
+#pragma unroll
+      for (int m = 0; m < MT; ++m)
+#pragma unroll
+        for (int f = 0; f < NF; ++f)
+          part[wave - half][m * NF + f][lane] = acc[m][f];
+    __syncthreads();
+    if (wave < half)
+#pragma unroll
+      for (int m = 0; m < MT; ++m)
+#pragma unroll
+        for (int f = 0; f < NF; ++f) {
+          const f32x4 p = part[wave][m * NF + f][lane];
+#pragma unroll
+          for (int r = 0; r < 4; ++r) acc[m][f][r] += p[r];
+        }
+    __syncthreads();
+  }
+  if (wave != 0) return;
 #pragma unroll
   for (int m = 0; m < MT; ++m)
 #pragma unroll
-    for (int f = 0; f < 4; ++f) part[wave][m * 4 + f][lane] = acc[m][f];
-  __syncthreads();
-  auto total = [&](int q) {
-    f32x4 a = part[0][q][lane];
-#pragma unroll
-    for (int v = 1; v < 4; ++v) {
-      const f32x4 p = part[v][q][lane];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) a[r] += p[r];
-    }
-    return a;
-  };
-  if constexpr (GLU) {
-    for (int q = wave; q < MT * 2; q += 4) { // (row fragment, column fragment)
-      const int m = q >> 1, f = q & 1;
-      const f32x4 gt = total(m * 4 + f), up = total(m * 4 + 2 + f);
+    for (int f = 0; f < NC; ++f) {
       const int i = n0 + f * 16 + c;
       if (i >= N) continue;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int t = m0 + m * 16 + hi * 4 + r;
         if (t >= T) continue;
-        const float s = we[(int64_t)t * E + e];
-        const float g = gt[r] * s;
-        out[((int64_t)e * T + t) * N + i] =
-            f2bits(g * __builtin_amdgcn_rcpf(1.f + __expf(-g)) * (up[r] * s));
+        float v = acc[m][f][r];
+        if constexpr (GLU) {
+          const float s = we[(int64_t)t * E + e];
+          const float g = v * s;
+          v = g * __builtin_amdgcn_rcpf(1.f + __expf(-g)) *
+              (acc[m][NC + f][r] * s);
+        } else if constexpr (KIND == kReluSq) {
+          v = fmaxf(v, 0.f);
+          v = v * v;
+        }
+        out[((int64_t)e * T + t) * N + i] = f2bits(v);
       }
     }
-  } else {
-    for (int q = wave; q < MT * 4; q += 4) {
-      const int m = q >> 2, f = q & 3;
-      const f32x4 a = total(q);
-      const int i = n0 + f * 16 + c;
-      if (i >= N) continue;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = m0 + m * 16 + hi * 4 + r;
-        if (t < T) out[((int64_t)e * T + t) * N + i] = f2bits(a[r]);
-      }
-    }
-  }
 }
 
 // ---- merge ----------------------------------------------------------------------
@@ -410,8 +441,9 @@ void moe_router(c10::optional<torch::Tensor> x, torch::Tensor w,
   if (x.has_value()) {
     DNET_CHECK(x->dim() == 2 && x->is_contiguous() && x->size(0) == T &&
                    x->size(1) == W, "x [T, W]");
-    if (is_bf16(*x)) MR(short, 256, (const short*)x->data_ptr(), nullptr);
-    else if (is_f32(*x)) MR(float, 256, (const float*)x->data_ptr(), nullptr);
+    const int nt = 64 * std::min(R, 16);
+    if (is_bf16(*x)) MR(short, nt, (const short*)x->data_ptr(), nullptr);
+    else if (is_f32(*x)) MR(float, nt, (const float*)x->data_ptr(), nullptr);
     else DNET_CHECK(false, "moe_router: dtype");
   } else {
     DNET_CHECK(logits->dim() == 2 && is_f32(*logits) &&
@@ -467,25 +499,33 @@ void moe_gather(torch::Tensor x, torch::Tensor order, torch::Tensor val,
 
 static void rows_launch(const torch::Tensor& x, const torch::Tensor& w,
                         const torch::Tensor& we, torch::Tensor& out, int64_t T,
-                        int64_t K, int64_t N, bool glu, int64_t x_expert) {
+                        int64_t K, int64_t N, int kind, int64_t x_expert) {
   const int64_t E = we.size(1);
-  const int mt = T <= 16 ? 1 : (T <= 32 ? 2 : 4);
-  const dim3 grid((unsigned)cdiv(N, glu ? 32 : 64),
-                  (unsigned)cdiv(T, 16 * mt), (unsigned)E);
   auto st = current_stream();
-#define RL(MM, GG)                                                            \
-  hipLaunchKernelGGL((moe_rows_kernel<MM, GG>), grid, dim3(256), 0, st,       \
-                     (const short*)x.data_ptr(), (const short*)w.data_ptr(),  \
-                     we.data_ptr<float>(), (short*)out.data_ptr(), (int)K,    \
-                     (int)N, (int)E, (int)T, x_expert)
-#define RL_M(GG)                  \
-  do {                            \
-    if (mt == 1) RL(1, GG);       \
-    else if (mt == 2) RL(2, GG);  \
-    else RL(4, GG);               \
-  } while (0)
-  if (glu) RL_M(true); else RL_M(false);
-#undef RL_M
+#define RL(MM, NF, NW, UU, GG)                                                \
+  hipLaunchKernelGGL((moe_rows_kernel<MM, NF, NW, UU, GG>),                   \
+                     dim3((unsigned)cdiv(N, GG == kGlu ? NF * 8 : NF * 16),           \
+                          (unsigned)cdiv(T, 16 * MM), (unsigned)E),           \
+                     dim3(NW * 64), 0, st, (const short*)x.data_ptr(),        \
+                     (const short*)w.data_ptr(), we.data_ptr<float>(),        \
+                     (short*)out.data_ptr(), (int)K, (int)N, (int)E, (int)T,  \
+                     x_expert)
+  // shapes measured at 4096 x 3072 experts: few rows want more workgroups
+  // (narrow column tiles), more rows wider tiles per pass over the rows
+  if (T <= 16) {
+    if (kind == kGlu) RL(1, 2, 8, 4, kGlu);
+    else if (kind == kReluSq) RL(1, 2, 8, 8, kReluSq);
+    else if (T <= 2) RL(1, 1, 8, 4, kPlain);
+    else RL(1, 2, 8, 8, kPlain);
+  } else if (T <= 32) {
+    if (kind == kGlu) RL(2, 4, 8, 4, kGlu);
+    else if (kind == kReluSq) RL(2, 4, 4, 4, kReluSq);
+    else RL(2, 4, 4, 4, kPlain);
+  } else {
+    if (kind == kGlu) RL(4, 4, 4, 2, kGlu);
+    else if (kind == kReluSq) RL(4, 4, 4, 2, kReluSq);
+    else RL(4, 4, 4, 2, kPlain);
+  }
 #undef RL
 }
 
@@ -502,7 +542,22 @@ void moe_gateup_rows(torch::Tensor x, torch::Tensor w, torch::Tensor we,
                  act.size(1) == T && act.size(2) == N && K % 8 == 0 && K > 0 &&
                  N > 0, "moe_gateup_rows: shapes");
   if (T == 0) return;
-  rows_launch(x, w, we, act, T, K, N, true, 0);
+  rows_launch(x, w, we, act, T, K, N, kGlu, 0);
+}
+
+void moe_up_rows(torch::Tensor x, torch::Tensor w, torch::Tensor we,
+                 torch::Tensor act) {
+  const int64_t T = x.size(0), K = x.size(1), E = w.size(0), N = w.size(1);
+  DNET_CHECK(is_bf16(x) && is_bf16(w) && is_bf16(act) && is_f32(we) &&
+                 x.is_contiguous() && w.is_contiguous() &&
+                 act.is_contiguous() && we.is_contiguous(),
+             "moe_up_rows: contiguous bf16, we fp32");
+  DNET_CHECK(x.dim() == 2 && w.dim() == 3 && w.size(2) == K && we.dim() == 2 &&
+                 we.size(0) == T && we.size(1) == E && act.dim() == 3 &&
+                 act.size(0) == E && act.size(1) == T && act.size(2) == N &&
+                 K % 8 == 0 && K > 0 && N > 0, "moe_up_rows: shapes");
+  if (T == 0) return;
+  rows_launch(x, w, we, act, T, K, N, kReluSq, 0);
 }
 
 void moe_down_rows(torch::Tensor act, torch::Tensor w, torch::Tensor we,
@@ -519,7 +574,7 @@ void moe_down_rows(torch::Tensor act, torch::Tensor w, torch::Tensor we,
                  y.size(1) == T && y.size(2) == N && K % 8 == 0 && K > 0,
              "moe_down_rows: shapes");
   if (T == 0) return;
-  rows_launch(act, w, we, y, T, K, N, false, T * K);
+  rows_launch(act, w, we, y, T, K, N, kPlain, T * K);
 }
 
 void moe_merge(torch::Tensor y, torch::Tensor at,

@@ -133,14 +133,14 @@ bool is_f32(const torch::Tensor& t) { return t.scalar_type() == torch::kFloat32;
 // (its norm is recomputed), the slot's state, or zero at position 0. With
 // `a` (one token per row): x += rms(a) * wa first.
 template <typename T, int V, bool RES>
-__global__ __launch_bounds__(256) void norm_shift_kernel(
+__global__ __launch_bounds__(1024) void norm_shift_kernel(
     float* __restrict__ x, const T* __restrict__ a,
     const float* __restrict__ wa, const float* __restrict__ wn,
     const float* __restrict__ mu, float* prev, T* __restrict__ y,
     const Rows g, const int W, const float eps, const int strip,
     const int write_state) {
   extern __shared__ __attribute__((aligned(16))) float hp[];    // [W]
-  __shared__ float red[8];
+  __shared__ float red[16];
   const int nstrip = (g.T + strip - 1) / strip;
   const int b = blockIdx.x / nstrip;
   const int t0 = (blockIdx.x % nstrip) * strip;
@@ -448,10 +448,12 @@ void norm_token_shift(torch::Tensor x, c10::optional<torch::Tensor> a,
   while (strip > 4 && B * ((T + strip - 1) / strip) < 512) strip /= 2;
   const int nstrip = (int)((T + strip - 1) / strip);
   const bool v4 = W % 4 == 0;
+  // decode: few workgroups, so more waves on each row
+  const int nt = T == 1 && W >= 4096 ? 1024 : (T == 1 && W >= 1024 ? 512 : 256);
   auto st = current_stream();
 #define NS(TT, VV, RR)                                                        \
   hipLaunchKernelGGL((norm_shift_kernel<TT, VV, RR>),                         \
-                     dim3((unsigned)(B * nstrip)), dim3(256), lds, st,        \
+                     dim3((unsigned)(B * nstrip)), dim3(nt), lds, st,         \
                      x.data_ptr<float>(),                                     \
                      RR ? (const TT*)a->data_ptr() : nullptr,                 \
                      RR ? wa->data_ptr<float>() : nullptr,                    \

@@ -203,12 +203,16 @@ def test_expert_row_kernels(T, W, I, E, top):
         assert not bool((idx == 0).any())
     act = ops.moe_gateup_rows(x, w1, we)
     want = ref.moe_gateup_rows(x.cpu(), w1.cpu(), we.cpu())
+    up = ops.moe_up_rows(x, w1, we)      # ungated, squared ReLU
+    wu = ref.moe_up_act(x.cpu(), w1.cpu(), we.cpu())
     y = ops.moe_down_rows(act, w2, we)
     wy = ref.moe_down_rows(act.cpu(), w2.cpu(), we.cpu())
     for e in range(E):
         rows = (idx == e).any(dim=1).cpu()
         torch.testing.assert_close(act[e].cpu().float()[rows],
                                    want[e].float()[rows], **_tol(dt))
+        torch.testing.assert_close(up[e].cpu().float()[rows],
+                                   wu[e].float()[rows], **_tol(dt))
         torch.testing.assert_close(y[e].cpu().float()[rows],
                                    wy[e].float()[rows], **_tol(dt))
     out = ops.moe_merge(y, idx, None, None, dt)
