@@ -660,6 +660,8 @@ def turevik_config(width: int, vocab: int, pattern: str = "lsg",
         c = pattern[i % len(pattern)]
         if c == "g":
             kind, m = "mingru", {"width": gru_width or width}
+        elif c not in "ls" or (c == "s" and own is None):
+            raise ValueError(f"turevik_config: pattern {pattern!r}")
         else:
             kind = "latent_attention"
             m = {"heads": heads, "dim": dim, "rot_dim": rot_dim,
