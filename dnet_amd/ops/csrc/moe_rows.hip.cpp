@@ -222,11 +222,11 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(
 }
 
 // ---- experts on the rows of a decode batch ----------------------------------------
-// grid (column tiles, row blocks of 16 MT, E), NW waves. A wave owns every
-// NW-th 32-wide step of the inner dimension (the waves read neighbouring
-// pieces of the same weight rows), NF weight fragments x MT row fragments of
-// v_mfma_f32_16x16x32_bf16, U steps in flight; the partial sums fold wave by
-// wave through LDS. GLU: the first half of the fragments are gate columns,
+// grid (column tiles, row blocks of 16 MT, E), NW waves. The inner
+// dimension goes in groups of NW x U 32-wide steps, U neighbouring ones per
+// wave (64 U bytes of every weight row it reads), NF weight fragments x MT row fragments of
+// v_mfma_f32_16x16x32_bf16, the next group in flight while one is multiplied;
+// the partial sums fold wave by wave through LDS. GLU: the first half of the fragments are gate columns,
 // the second half the up columns beside them (8 NF columns of act), inputs
 // scaled by the routing weight; else 16 NF plain or squared-ReLU columns.
 constexpr int kPlain = 0, kGlu = 1, kReluSq = 2;
@@ -269,32 +269,34 @@ __global__ __launch_bounds__(NW * 64) void moe_rows_kernel(
     for (int f = 0; f < NF; ++f) acc[m][f] = {0.f, 0.f, 0.f, 0.f};
 
   const int full = K / 32;                   // whole steps
-  // C steps s, s + NW, ... of this wave; `in`: the lane's 8 entries exist
-  auto run = [&](const int s, const bool in, auto cnt) {
-    constexpr int C = decltype(cnt)::value;
-    bf16x8 wf[C][NF], xf[C][MT];
-    short8 z;
+  short8 z;
 #pragma unroll
-    for (int j = 0; j < 8; ++j) z.x[j] = 0;
-    const bf16x8 zero = *reinterpret_cast<const bf16x8*>(&z);
+  for (int j = 0; j < 8; ++j) z.x[j] = 0;
+  const bf16x8 zero = *reinterpret_cast<const bf16x8*>(&z);
+  struct Batch { bf16x8 wf[U][NF], xf[U][MT]; };
+  auto load = [&](Batch& q, const int s) {
+    // a row's neighbouring 64 B pieces back to back
 #pragma unroll
-    for (int u = 0; u < C; ++u) {
-      const int at = (s + NW * u) * 32;
+    for (int f = 0; f < NF; ++f)
 #pragma unroll
-      for (int f = 0; f < NF; ++f)
-        wf[u][f] = in ? *reinterpret_cast<const bf16x8*>(wp[f] + at) : zero;
+      for (int u = 0; u < U; ++u)
+        q.wf[u][f] =
+            *reinterpret_cast<const bf16x8*>(wp[f] + (s + u) * 32);
 #pragma unroll
-      for (int m = 0; m < MT; ++m)
-        xf[u][m] = in ? *reinterpret_cast<const bf16x8*>(xp[m] + at) : zero;
-    }
+    for (int m = 0; m < MT; ++m)
 #pragma unroll
-    for (int u = 0; u < C; ++u)
+      for (int u = 0; u < U; ++u)
+        q.xf[u][m] = *reinterpret_cast<const bf16x8*>(xp[m] + (s + u) * 32);
+  };
+  auto mul = [&](const Batch& q) {
+#pragma unroll
+    for (int u = 0; u < U; ++u)
 #pragma unroll
       for (int m = 0; m < MT; ++m)
 #pragma unroll
         for (int f = 0; f < NF; ++f)
           acc[m][f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              xf[u][m], wf[u][f], acc[m][f], 0, 0, 0);
+              q.xf[u][m], q.wf[u][f], acc[m][f], 0, 0, 0);
   };
   // every workgroup starts at another place of the inner dimension: weight
   // rows are often a power of two apart, and workgroups in step would all
@@ -302,16 +304,43 @@ __global__ __launch_bounds__(NW * 64) void moe_rows_kernel(
   const int groups = full / (NW * U);
   const int turn =
       groups > 1 ? (int)((blockIdx.x * 5 + blockIdx.z * 3) % groups) : 0;
-  for (int g = 0; g < groups; ++g) {
-    int gg = g + turn;
-    if (gg >= groups) gg -= groups;
-    run(gg * NW * U + wave, true, std::integral_constant<int, U>{});
+  auto place = [&](int g) {
+    g += turn;
+    if (g >= groups) g -= groups;
+    return (g * NW + wave) * U;
+  };
+  if (groups > 0) {
+    Batch q0, q1;
+    load(q0, place(0));
+    int g = 0;
+    for (; g + 2 <= groups; g += 2) {
+      load(q1, place(g + 1));
+      __builtin_amdgcn_sched_barrier(0);
+      mul(q0);
+      if (g + 2 < groups) load(q0, place(g + 2));
+      __builtin_amdgcn_sched_barrier(0);
+      mul(q1);
+    }
+    if (g < groups) mul(q0);
   }
-  for (int s0 = groups * NW * U + wave; s0 < full; s0 += NW)
-    run(s0, true, std::integral_constant<int, 1>{});
+  auto tail = [&](const int s, const bool in) {
+    bf16x8 wf[NF], xf[MT];
+#pragma unroll
+    for (int f = 0; f < NF; ++f)
+      wf[f] = in ? *reinterpret_cast<const bf16x8*>(wp[f] + s * 32) : zero;
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+      xf[m] = in ? *reinterpret_cast<const bf16x8*>(xp[m] + s * 32) : zero;
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+      for (int f = 0; f < NF; ++f)
+        acc[m][f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xf[m], wf[f],
+                                                            acc[m][f], 0, 0, 0);
+  };
+  for (int s = groups * NW * U + wave; s < full; s += NW) tail(s, true);
   if (full * 32 < K && wave == full % NW)    // the last, shorter step
-    run(full, full * 32 + hi * 8 < K,        // (K is a multiple of 8)
-        std::integral_constant<int, 1>{});
+    tail(full, full * 32 + hi * 8 < K);      // (K is a multiple of 8)
 
 #pragma unroll
   for (int half = NW / 2; half > 0; half >>= 1) {
@@ -510,22 +539,19 @@ static void rows_launch(const torch::Tensor& x, const torch::Tensor& w,
                      (const short*)w.data_ptr(), we.data_ptr<float>(),        \
                      (short*)out.data_ptr(), (int)K, (int)N, (int)E, (int)T,  \
                      x_expert)
-  // shapes measured at 4096 x 3072 experts: few rows want more workgroups
-  // (narrow column tiles), more rows wider tiles per pass over the rows
-  if (T <= 16) {
-    if (kind == kGlu) RL(1, 2, 8, 4, kGlu);
-    else if (kind == kReluSq) RL(1, 2, 8, 8, kReluSq);
-    else if (T <= 2) RL(1, 1, 8, 4, kPlain);
-    else RL(1, 2, 8, 8, kPlain);
-  } else if (T <= 32) {
-    if (kind == kGlu) RL(2, 4, 8, 4, kGlu);
-    else if (kind == kReluSq) RL(2, 4, 4, 4, kReluSq);
-    else RL(2, 4, 4, 4, kPlain);
-  } else {
-    if (kind == kGlu) RL(4, 4, 4, 2, kGlu);
-    else if (kind == kReluSq) RL(4, 4, 4, 2, kReluSq);
-    else RL(4, 4, 4, 2, kPlain);
-  }
+  // shapes measured at experts of 4096 x 3072 to 5120 x 12800: few rows want
+  // more workgroups (narrow column tiles)
+#define RL_K(MM, NF, NW, UU)                            \
+  do {                                                  \
+    if (kind == kGlu) RL(MM, NF, NW, UU, kGlu);         \
+    else if (kind == kReluSq) RL(MM, NF, NW, UU, kReluSq); \
+    else RL(MM, NF, NW, UU, kPlain);                    \
+  } while (0)
+  if (T <= 2 && kind == kPlain) RL(1, 1, 8, 4, kPlain);
+  else if (T <= 16) RL_K(1, 2, 8, 4);
+  else if (T <= 32) RL_K(2, 4, 4, 2);
+  else RL_K(4, 4, 4, 2);
+#undef RL_K
 #undef RL
 }
 
