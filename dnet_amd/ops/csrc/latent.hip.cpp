@@ -63,7 +63,8 @@ __global__ __launch_bounds__(256) void latent_append_kernel(
 }
 
 // grid (B*T); q [M, ld >= H*(d+rd)], qabs [H, M, R] -> out [M, H*(R+rd)]
-template <typename T>
+// V entries (16 B, or one) per access to the part that is copied
+template <typename T, int V>
 __global__ __launch_bounds__(256) void latent_q_pack_kernel(
     const T* __restrict__ q, const int64_t ld, const T* __restrict__ qabs,
     const float* __restrict__ freq, const int* __restrict__ pos,
@@ -79,9 +80,15 @@ __global__ __launch_bounds__(256) void latent_q_pack_kernel(
   const int rd = 2 * np, D = R + rd;
   const T* qr = q + row * ld;
   T* orow = out + row * (int64_t)H * D;
-  for (int idx = threadIdx.x; idx < H * R; idx += blockDim.x) {
-    const int h = idx / R, i = idx % R;
-    orow[(int64_t)h * D + i] = qabs[((int64_t)h * M + row) * R + i];
+  const int RV = R / V;
+  for (int idx = threadIdx.x; idx < H * RV; idx += blockDim.x) {
+    const int h = idx / RV, i = (idx % RV) * V;
+    const T* src = qabs + ((int64_t)h * M + row) * R + i;
+    T* dst = orow + (int64_t)h * D + i;
+    if constexpr (V * sizeof(T) == 16)
+      *reinterpret_cast<int4*>(dst) = *reinterpret_cast<const int4*>(src);
+    else
+      *dst = *src;
   }
   for (int idx = threadIdx.x; idx < H * np; idx += blockDim.x) {
     const int h = idx / np, i = idx % np;
@@ -164,16 +171,21 @@ void latent_q_pack(torch::Tensor q, torch::Tensor qabs, torch::Tensor rot_freq,
                  pos.numel() >= M / T, "pos int32 [B]");
   if (M == 0) return;
   auto st = current_stream();
-#define LQ(TT)                                                               \
-  hipLaunchKernelGGL((latent_q_pack_kernel<TT>), dim3((unsigned)M),          \
+  const int64_t D = R + 2 * np;
+#define LQ(TT, VV)                                                           \
+  hipLaunchKernelGGL((latent_q_pack_kernel<TT, VV>), dim3((unsigned)M),      \
                      dim3(256), 0, st, (const TT*)q.data_ptr(), q.size(1),   \
                      (const TT*)qabs.data_ptr(),                             \
                      rot_freq.data_ptr<float>(), pos.data_ptr<int>(),        \
                      (TT*)out.data_ptr(), (int)T, M, (int)H, (int)d,         \
                      (int)np, (int)R)
-  if (q.scalar_type() == torch::kBFloat16) LQ(short);
-  else if (q.scalar_type() == torch::kFloat32) LQ(float);
-  else DNET_CHECK(false, "latent_q_pack: dtype");
+  if (q.scalar_type() == torch::kBFloat16) {
+    if (R % 8 == 0 && D % 8 == 0) LQ(short, 8); else LQ(short, 1);
+  } else if (q.scalar_type() == torch::kFloat32) {
+    if (R % 4 == 0 && D % 4 == 0) LQ(float, 4); else LQ(float, 1);
+  } else {
+    DNET_CHECK(false, "latent_q_pack: dtype");
+  }
 #undef LQ
 }
 
