@@ -20,8 +20,9 @@ Mixers (``cfg.layer_specs[l]["type"]``):
   learned sink per head in the denominator. A layer with ``kv_from`` = j owns
   no rows: it reads those of the earlier layer j with its own queries,
   up-projections and sinks.
-* ``mingru``: a gated recurrence whose gates read the current token only,
-  S <- (1 - z) S + z * candidate per channel, output gated by silu.
+* ``mingru``: S <- (1 - z) S + z * candidate per channel, with z and the
+  candidate computed from the step's input alone (no state feedback, so a
+  prompt is a scan of affine maps); output gated by silu.
 
 Feed-forwards: dense (gelu-gated) or a mixture of silu-gated experts: sigmoid
 router, the largest ``top`` scores kept as they are, each score multiplying

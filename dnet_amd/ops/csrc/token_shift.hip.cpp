@@ -4,8 +4,9 @@
 //                     previous token's h; optionally x += rms(a) * wa first
 //                     (decode steps: residual update, norm and shift in one
 //                     launch). The slot's last h is its state (fp32).
-//   mingru_scan       S <- (1 - z) S + z * candidate per channel, gates from
-//                     the current token only; y = S * silu(gate)
+//   mingru_scan       S <- (1 - z) S + z * candidate per channel, z and the
+//                     candidate from the step's projections alone (no state
+//                     feedback); y = S * silu(gate)
 //   cache_append      projection columns as they are into cache rows
 //   gated_act         act(s gate) * (s up) over [gate | up] rows, act = silu
 //                     or tanh-gelu, s an optional factor per row

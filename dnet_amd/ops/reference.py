@@ -1261,8 +1261,8 @@ def mingru_scan(src: torch.Tensor, z0: int, x0: int, g0: int,
                 bz: torch.Tensor, bx: torch.Tensor, state: torch.Tensor,
                 pos: torch.Tensor, T: int, lens=None,
                 slots=None) -> torch.Tensor:
-    """Gated recurrence whose gates read the current token only, fp32. With
-    N = len(bz) and columns z0 / x0 / g0 of src [B*T, ld]: z = sigmoid(zc +
+    """Per-channel blend of state and candidate, both functions of the step's
+    own projections (no feedback from the state), fp32. With N = len(bz) and columns z0 / x0 / g0 of src [B*T, ld]: z = sigmoid(zc +
     bz), u = xc + bx, candidate = u + 1/2 where u >= 0 and sigmoid(u)
     elsewhere; S <- (1 - z) S + z * candidate; y = S * silu(gc), in src's
     dtype. ``state`` fp32 [Bc, N] per slot: zero at position 0, advanced by

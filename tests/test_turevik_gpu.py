@@ -180,7 +180,7 @@ def test_router_plan_gather_merge(dt, T, W, E, top, sg):
 
 
 @pytest.mark.parametrize("T,W,I,E,top", [(1, 64, 32, 5, 1), (7, 72, 40, 6, 2),
-                                         (16, 320, 64, 12, 1),
+                                         (16, 352, 72, 11, 1),
                                          (32, 1024, 512, 8, 2),
                                          (33, 200, 24, 3, 3),
                                          (64, 136, 104, 4, 1),
@@ -222,7 +222,7 @@ def test_expert_row_kernels(T, W, I, E, top):
 
 
 @pytest.mark.parametrize("dt", DTS)
-@pytest.mark.parametrize("H,R,rd", [(4, 96, 32), (3, 20, 6), (16, 64, 32),
+@pytest.mark.parametrize("H,R,rd", [(5, 88, 24), (3, 20, 6), (16, 64, 32),
                                     (32, 192, 64)])
 def test_sink_on_shared_rows(dt, H, R, rd):
     """Attention against shared latent rows with a sink that matters, in

@@ -105,7 +105,8 @@ def latent_attention(h, p, m, eps, shared=None):
 
 
 def mingru(h, p, m, eps):
-    """Gated recurrence whose gates read the current token only."""
+    """S_t = (1 - z_t) S_(t-1) + z_t c_t per channel; no state feedback into
+    z and c."""
     z = sigmoid(h @ p["z"].T + p["z.b"])
     u = h @ p["x"].T + p["x.b"]
     cand = torch.where(u >= 0, u + 0.5, sigmoid(u))
