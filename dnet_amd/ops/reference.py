@@ -1261,10 +1261,11 @@ def mingru_scan(src: torch.Tensor, z0: int, x0: int, g0: int,
                 bz: torch.Tensor, bx: torch.Tensor, state: torch.Tensor,
                 pos: torch.Tensor, T: int, lens=None,
                 slots=None) -> torch.Tensor:
-    """Per-channel blend of state and candidate, both functions of the step's
-    own projections (no feedback from the state), fp32. With N = len(bz) and columns z0 / x0 / g0 of src [B*T, ld]: z = sigmoid(zc +
-    bz), u = xc + bx, candidate = u + 1/2 where u >= 0 and sigmoid(u)
-    elsewhere; S <- (1 - z) S + z * candidate; y = S * silu(gc), in src's
+    """Per-channel blend of the state with a candidate, fp32; blend and
+    candidate come from the step's own projections (no feedback from the
+    state). With N = len(bz) and columns z0 / x0 / g0 of src [B*T, ld]:
+    z = sigmoid(zc + bz), u = xc + bx, candidate = u + 1/2 where u >= 0 and
+    sigmoid(u) elsewhere; S <- (1 - z) S + z * candidate; y = S * silu(gc), in src's
     dtype. ``state`` fp32 [Bc, N] per slot: zero at position 0, advanced by
     the rows' real tokens. Padding rows of y are zero."""
     M, N = src.shape[0], bz.numel()
