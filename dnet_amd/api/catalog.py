@@ -50,6 +50,8 @@ model_catalog: list[CatalogEntry] = [
                  tokenizer="byte", ci_test=True),
     CatalogEntry("turevik-tiny-random", preset="turevik-tiny",
                  tokenizer="byte", ci_test=True),
+    CatalogEntry("fedinex-tiny-random", preset="fedinex-tiny",
+                 tokenizer="byte", ci_test=True),
     CatalogEntry("openai/gpt-oss-20b", repo="openai/gpt-oss-20b"),
     CatalogEntry("deepseek-ai/DeepSeek-V2-Lite", repo="deepseek-ai/DeepSeek-V2-Lite"),
     # real checkpoints (local safetensors dir or pre-downloaded HF cache)

@@ -59,5 +59,9 @@ from .turevik import TurevikRingModel  # noqa: E402
 
 register(TurevikRingModel)
 
-__all__ = ["GegoraxRingModel", "KomizenRingModel", "LurisunRingModel", "ModelConfig", "QuantConfig", "RingModel", "MoERingModel", "KVCache", "PosudraRingModel",
+from .fedinex import FedinexRingModel  # noqa: E402
+
+register(FedinexRingModel)
+
+__all__ = ["FedinexRingModel", "GegoraxRingModel", "KomizenRingModel", "LurisunRingModel", "ModelConfig", "QuantConfig", "RingModel", "MoERingModel", "KVCache", "PosudraRingModel",
            "TurevikRingModel", "Linear", "PRESETS", "get_ring_model", "register"]

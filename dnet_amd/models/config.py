@@ -429,8 +429,103 @@ class ModelConfig:
         )
 
     @classmethod
+    def from_fedinex(cls, cfg: dict,
+                     quant: Optional[QuantConfig] = None) -> "ModelConfig":
+        """Fedinex checkpoints list their layers: {"architecture":
+        "Fedinex", "vocab", "width", "norm": {"eps"}, "layers": [{"type":
+        "attention" | "parallel" | "gla", "mixer": {...}, "mlp": {"kind":
+        "dense", "ff", "limit"} | {"kind": "moe", "router": {"experts",
+        "top", "scale", "groups": {"count", "keep"} (optional)}, "expert":
+        {"ff", "limit"}} | null}, ...]}. A parallel mixer holds a convolved
+        attention ("left") and a matrix memory ("right") with one output
+        factor each. Every size and constant is per layer."""
+        attn = ("heads", "kv_heads", "dim", "vdim", "scale")
+        need = {"attention": {"": attn},
+                "parallel": {"": ("left_scale", "right_scale"),
+                             "left": attn + ("conv",),
+                             "right": ("heads", "dim", "vdim", "gate_cap")},
+                "gla": {"": ("heads", "dim", "vdim", "tau")}}
+        specs = [dict(s) for s in cfg["layers"]]
+        mixed = None                    # value width of the mixing layers
+        for i, s in enumerate(specs):
+            kind, m = s.get("type"), s.get("mixer") or {}
+            if kind not in need:
+                raise ValueError(f"fedinex layer {i}: unknown mixer type "
+                                 f"{kind!r}")
+            for side, keys in need[kind].items():
+                part = m.get(side) or {} if side else m
+                missing = [k for k in keys if k not in part]
+                if missing:
+                    raise ValueError(f"fedinex layer {i}: mixer "
+                                     f"{side} lacks {missing}")
+            at = m if kind == "attention" else m.get("left")
+            if at is not None:
+                if at["heads"] % at["kv_heads"]:
+                    raise ValueError(f"fedinex layer {i}: heads % kv_heads")
+                rot = at.get("rot")
+                if rot and (int(rot["dims"]) % 2
+                            or int(rot["dims"]) > at["dim"]):
+                    raise ValueError(f"fedinex layer {i}: rot.dims must be "
+                                     "even and at most dim")
+            if kind == "parallel" and int(at["conv"]) < 1:
+                raise ValueError(f"fedinex layer {i}: conv needs a tap")
+            if kind == "attention":
+                mask = m.get("mask")
+                if mask and (int(mask["size"]) < 1
+                             or int(mask.get("keep_first") or 0) < 0):
+                    raise ValueError(f"fedinex layer {i}: mask")
+                if m.get("v_mix"):
+                    mixed = mixed or (m["kv_heads"], m["vdim"])
+                    if mixed != (m["kv_heads"], m["vdim"]):
+                        raise ValueError(f"fedinex layer {i}: value-mixing "
+                                         "layers differ in their values")
+            ff = s.get("mlp")
+            if ff is None:
+                continue
+            if ff.get("kind") == "dense":
+                if "ff" not in ff or "limit" not in ff:
+                    raise ValueError(f"fedinex layer {i}: mlp lacks ff/limit")
+            elif ff.get("kind") == "moe":
+                r = ff["router"]
+                g = r.get("groups") or {"count": 1, "keep": 1}
+                E = int(r["experts"])
+                if E % g["count"] or not 1 <= g["keep"] <= g["count"] or \
+                        not 1 <= r["top"] <= g["keep"] * (E // g["count"]):
+                    raise ValueError(f"fedinex layer {i}: router groups/top")
+            else:
+                raise ValueError(f"fedinex layer {i}: unknown feed-forward "
+                                 f"kind {ff.get('kind')!r}")
+        att = next((s["mixer"] if s["type"] == "attention"
+                    else s["mixer"]["left"] for s in specs
+                    if s["type"] != "gla"), specs[0]["mixer"])
+        ffs = [s["mlp"] for s in specs if s.get("mlp") is not None]
+        moe = [f for f in ffs if f["kind"] == "moe"]
+        return cls(
+            model_type="fedinex",
+            hidden_size=cfg["width"],
+            num_layers=len(specs),
+            num_q_heads=att["heads"],
+            num_kv_heads=att.get("kv_heads", 1),
+            head_dim=att["dim"],
+            v_head_dim=att["vdim"],
+            intermediate_size=max((f["ff"] for f in ffs
+                                   if f["kind"] == "dense"), default=0),
+            num_experts=max((f["router"]["experts"] for f in moe), default=0),
+            num_experts_per_tok=max((f["router"]["top"] for f in moe),
+                                    default=0),
+            moe_intermediate_size=max((f["expert"]["ff"] for f in moe),
+                                      default=0),
+            vocab_size=cfg["vocab"],
+            rms_eps=cfg["norm"]["eps"],
+            layer_specs=specs,
+            quant=quant,
+        )
+
+    @classmethod
     def from_hf(cls, cfg: dict, quant: Optional[QuantConfig] = None) -> "ModelConfig":
         arch = str(cfg.get("architecture", "")).lower()
+        if arch == "fedinex" or cfg.get("model_type") == "fedinex":
+            return cls.from_fedinex(cfg, quant)
         if arch == "turevik" or cfg.get("model_type") == "turevik":
             return cls.from_turevik(cfg, quant)
         if arch == "lurisun" or cfg.get("model_type") == "lurisun":
@@ -684,6 +779,62 @@ def turevik_config(width: int, vocab: int, pattern: str = "lsg",
             "norm": {"eps": eps}, "layers": out}
 
 
+def fedinex_config(width: int, vocab: int, pattern: str = "apg",
+                   layers: int = 0, heads: int = 4, kv_heads: int = 2,
+                   dim: int = 32, vdim: int = 24, rot_dims: int = 16,
+                   window: int = 20, keep_first: int = 3, v_mix: bool = True,
+                   left_heads: int = 4, left_kv_heads: int = 2,
+                   left_dim: int = 32, left_vdim: int = 32, conv: int = 4,
+                   left_rot_dims: int = 16, mem_heads: int = 4,
+                   mem_dim: int = 16, mem_vdim: int = 32,
+                   gate_cap: float = 15.0, left_scale: float = 0.7,
+                   right_scale: float = 0.6, gla_heads: int = 4,
+                   gla_dim: int = 16, gla_vdim: int = 32, tau: float = 16.0,
+                   ff: int = 192, limit: float = 2.0, experts: int = 8,
+                   top: int = 2, expert_ff: int = 64, groups: int = 2,
+                   keep_groups: int = 1, router_scale: float = 1.5,
+                   rot_base: float = 10000.0, left_rot_base: float = 50000.0,
+                   eps: float = 1e-6) -> dict:
+    """A fedinex stack in the checkpoint's config.json layout. ``pattern``
+    repeats over ``layers`` layers (default: once): 'a' = windowed attention
+    with kept first tokens and value mixing, 'p' = convolved attention beside
+    a matrix memory, 'g' = gated linear attention. Every second layer's
+    feed-forward is a mixture of experts when ``experts`` > 0, dense
+    otherwise."""
+    att = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim,
+           "scale": dim ** -0.5, "v_mix": v_mix}
+    if window:
+        att["mask"] = {"size": window, "keep_first": keep_first}
+    if rot_dims:
+        att["rot"] = {"base": rot_base, "dims": rot_dims}
+    left = {"heads": left_heads, "kv_heads": left_kv_heads, "dim": left_dim,
+            "vdim": left_vdim, "scale": left_dim ** -0.5, "conv": conv}
+    if left_rot_dims:
+        left["rot"] = {"base": left_rot_base, "dims": left_rot_dims}
+    mix = {
+        "a": ("attention", att),
+        "p": ("parallel", {"left": left, "left_scale": left_scale,
+                           "right": {"heads": mem_heads, "dim": mem_dim,
+                                     "vdim": mem_vdim, "gate_cap": gate_cap},
+                           "right_scale": right_scale}),
+        "g": ("gla", {"heads": gla_heads, "dim": gla_dim, "vdim": gla_vdim,
+                      "tau": tau}),
+    }
+    dense = {"kind": "dense", "ff": ff, "limit": limit} if ff else None
+    router = {"experts": experts, "top": top, "scale": router_scale}
+    if groups:
+        router["groups"] = {"count": groups, "keep": keep_groups}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff, "limit": limit},
+           "router": router}
+    out = []
+    for i in range(layers or len(pattern)):
+        kind, m = mix[pattern[i % len(pattern)]]
+        out.append({"type": kind, "mixer": dict(m),
+                    "mlp": moe if experts and i % 2 else dense})
+    return {"architecture": "Fedinex", "vocab": vocab, "width": width,
+            "norm": {"eps": eps}, "layers": out}
+
+
 # Known configs for synthetic benchmarking (random-init weights; no network).
 PRESETS: dict[str, dict] = {
     "llama-3-8b": dict(model_type="llama", hidden_size=4096, num_hidden_layers=32,
@@ -754,6 +905,7 @@ PRESETS: dict[str, dict] = {
     "lurisun-tiny": lurisun_config(128, 256, "nla", layers=4,
                                    logit_scale=0.5),
     "turevik-tiny": turevik_config(128, 256, "lsgs", layers=4),
+    "fedinex-tiny": fedinex_config(128, 256, "apg", layers=4),
     "tiny": dict(model_type="llama", hidden_size=128, num_hidden_layers=4,
                  num_attention_heads=2, num_key_value_heads=2, head_dim=64,
                  intermediate_size=256, vocab_size=256, rope_theta=10000.0),

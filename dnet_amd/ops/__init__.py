@@ -516,7 +516,8 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
              temp=None, softcap: float = 0.0, dist_r1=None, dist_r2=None,
              sinks=None, window: int = 0, pool_k=None, pool_v=None,
              pool: int = 0, v_dim: int = 0, chunk: int = 0,
-             sig_bias=None) -> torch.Tensor:
+             sig_bias=None, keep: int = 0, gate=None, gate_col: int = 0,
+             gate_scale: float = 1.0, out=None) -> torch.Tensor:
     """Causal attention against the cache with per-head temperature, tanh
     soft cap, logarithmic distance penalty and a sink in the softmax
     denominator (each optional). One entry point for decode (T=1) and
@@ -528,7 +529,13 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
     entries of the key rows, which the kernels then stage once for both.
     ``chunk`` > 0: a query sees only the keys of its own block of ``chunk``
     positions (blocks count from position 0). ``sig_bias`` fp32 [Hq]: no
-    softmax, the weight of a visible key is sigmoid(score + sig_bias[h])."""
+    softmax, the weight of a visible key is sigmoid(score + sig_bias[h]).
+    ``keep`` > 0 (with a window): the first ``keep`` keys stay visible beside
+    the window. ``gate`` [B*T, ld]: head h's result times gate_scale *
+    sigmoid(gate[row, gate_col + h]), before it is rounded. ``out``: a column
+    range of a wider zero-filled buffer for the result."""
+    if keep:
+        assert window and not pool and not chunk
     if sig_bias is not None:
         assert sinks is None and not pool
     if pool:
@@ -540,14 +547,15 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
         Dv = vcache.shape[3] if vcache is not None else v_dim
         Hq = q.shape[1] // D
         # padded rows of a ragged batch are never written by the kernel
-        out = (torch.zeros if lens is not None else torch.empty)(
-            q.shape[0], Hq * Dv, dtype=q.dtype, device=q.device)
+        if out is None:
+            out = (torch.zeros if lens is not None else torch.empty)(
+                q.shape[0], Hq * Dv, dtype=q.dtype, device=q.device)
         splits, partials = 1, None
         if T == 1:
             # a windowed row scans at most window + pooled entries
             span = kcache.shape[2]
             if window:
-                span = min(span, window + 64
+                span = min(span, window + 64 + (keep + 64 if keep else 0)
                            + (pool_k.shape[2] if pool else 0))
             if chunk:
                 span = min(span, chunk + 64)
@@ -577,11 +585,13 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
                            sinks, window or 0, partials, splits,
                            pool_k if pool else None,
                            pool_v if pool else None, pool or 0, Dv,
-                           chunk or 0, sig_bias)
+                           chunk or 0, sig_bias, keep or 0, gate, gate_col,
+                           gate_scale)
         return out
     return ref.attn_mod(q, kcache, vcache, pos, T, scale, lens, slots, temp,
                         softcap, dist_r1, dist_r2, sinks, window, pool_k,
-                        pool_v, pool, v_dim, chunk, sig_bias)
+                        pool_v, pool, v_dim, chunk, sig_bias, keep, gate,
+                        gate_col, gate_scale, out)
 
 
 # ---- pooled-block caches, short convolutions, linear recurrences ----
@@ -639,14 +649,17 @@ def delta_scan(src, r0: int, k0: int, v0: int, a0: int, wl, w0, ab, state,
 
 def gated_group_rmsnorm(y, gate_src, gate_col0: int, w, groups: int,
                         eps: float, gate_act: str, gate_first: bool,
-                        out_dtype: torch.dtype) -> torch.Tensor:
+                        out_dtype: torch.dtype, out=None) -> torch.Tensor:
+    """``out``: a column range of a wider buffer that takes the result."""
     if y.is_cuda:
-        out = torch.empty(y.shape, dtype=out_dtype, device=y.device)
+        if out is None:
+            out = torch.empty(y.shape, dtype=out_dtype, device=y.device)
         _native().gated_group_rmsnorm(y, gate_src, gate_col0, w, out, groups,
                                       eps, gate_act == "silu", gate_first)
         return out
-    return ref.gated_group_rmsnorm(y, gate_src, gate_col0, w, groups, eps,
-                                   gate_act, gate_first, out_dtype)
+    r = ref.gated_group_rmsnorm(y, gate_src, gate_col0, w, groups, eps,
+                                gate_act, gate_first, out_dtype)
+    return r if out is None else out.copy_(r)
 
 
 _ACT_KINDS = {"relu_sq": 0, "tanh": 1}
@@ -690,7 +703,8 @@ def clamped_glu(gu: torch.Tensor, alpha: float, limit: float) -> torch.Tensor:
     if gu.is_cuda:
         y = torch.empty(gu.shape[0], gu.shape[1] // 2, dtype=gu.dtype,
                         device=gu.device)
-        _native().clamped_glu(gu, y, alpha, limit)
+        _native().gated_act(gu.contiguous(), None, y, _GATED_ACTS["clamped"],
+                            alpha, limit)
         return y
     return ref.clamped_glu(gu, alpha, limit)
 
@@ -933,27 +947,32 @@ def cache_append(src, col0: int, cache, pos, T: int, lens=None,
     ref.cache_append(src, col0, cache, pos, T, lens, slots)
 
 
-_GATED_ACTS = {"silu": 0, "gelu_tanh": 1}
+_GATED_ACTS = {"silu": 0, "gelu_tanh": 1, "clamped": 2}
 
 
-def gated_act(gu, act: str, scale=None) -> torch.Tensor:
-    """[gate | up] -> act(s gate) * (s up), s the row's ``scale`` (or 1)."""
+def gated_act(gu, act: str, scale=None, alpha: float = 1.0,
+              limit: float = 0.0) -> torch.Tensor:
+    """[gate | up] -> act(s gate) * (s up), s the row's ``scale`` (or 1);
+    "clamped": g sigmoid(alpha g) (u + 1) s with g = min(gate, limit), u = up
+    clamped to +-limit."""
     if gu.is_cuda:
         y = torch.empty(gu.shape[0], gu.shape[1] // 2, dtype=gu.dtype,
                         device=gu.device)
-        _native().gated_act(gu, scale, y, _GATED_ACTS[act])
+        _native().gated_act(gu, scale, y, _GATED_ACTS[act], alpha, limit)
         return y
-    return ref.gated_act(gu, act, scale)
+    return ref.gated_act(gu, act, scale, alpha, limit)
 
 
 # rows up to which the router's products run inside the routing kernel
 _ROUTER_FUSED_ROWS = 128
 
 
-def moe_router(x, w, E: int, top: int):
+def moe_router(x, w, E: int, top: int, correction=None, groups: int = 1,
+               keep: int = 1, scale: float = 1.0):
     """Sigmoid router in fp32 with an optional shared-expert gate as the last
-    row of w [E (+1), W]: (idx, val, we, gate), see the reference. No host
-    sync."""
+    row of w [E (+1), W]: (idx, val, we, gate), see the reference. Optional
+    choice by score + ``correction`` among the ``keep`` best of ``groups``
+    groups; values times ``scale``. No host sync."""
     if x.is_cuda:
         T = x.shape[0]
         idx = torch.empty(T, top, dtype=torch.int32, device=x.device)
@@ -962,12 +981,13 @@ def moe_router(x, w, E: int, top: int):
         gate = (torch.empty(T, dtype=torch.float32, device=x.device)
                 if w.shape[0] > E else None)
         if T <= _ROUTER_FUSED_ROWS:
-            _native().moe_router(x, w, None, idx, val, we, gate)
+            _native().moe_router(x, w, None, idx, val, we, gate, correction,
+                                 groups, keep, scale)
         else:
             _native().moe_router(None, w, x.float() @ w.t(), idx, val, we,
-                                 gate)
+                                 gate, correction, groups, keep, scale)
         return idx, val, we, gate
-    return ref.moe_router(x, w, E, top)
+    return ref.moe_router(x, w, E, top, correction, groups, keep, scale)
 
 
 def moe_plan(idx, E: int):
@@ -1040,3 +1060,76 @@ def moe_merge(y, at, shared, gate, out_dtype: torch.dtype) -> torch.Tensor:
         _native().moe_merge(y, at, shared, gate, out)
         return out
     return ref.moe_merge(y, at, shared, gate, out_dtype)
+
+
+def moe_clamped_rows(x, w, we, alpha: float, limit: float) -> torch.Tensor:
+    """``moe_gateup_rows`` for clamped gated experts whose routing weight is a
+    factor of the result."""
+    if x.is_cuda:
+        E, I2, _ = w.shape
+        act = torch.empty(E, x.shape[0], I2 // 2, dtype=x.dtype,
+                          device=x.device)
+        _native().moe_clamped_rows(x, w, we, act, alpha, limit)
+        return act
+    return ref.moe_clamped_rows(x, w, we, alpha, limit)
+
+
+# ---- biased / convolved attention projections, gated linear attention, matrix
+# memory (fedinex) ----
+# csrc/qkv_rope.hip.cpp, csrc/linear_scan.hip.cpp. Angles, rotation, gates,
+# decays and recurrent states are fp32 whatever the activation dtype.
+
+def qkv_rope_append(src, col0: int, nq: int, nkv: int, d: int, dv: int,
+                    kcache, vcache, pos, T: int, lens=None, slots=None,
+                    bias=None, conv_w=None, conv_state=None, rot_freq=None,
+                    half: bool = False, vf=None, lam=None) -> torch.Tensor:
+    """q/k/v columns of a projection to attention operands (bias or short
+    convolution, rotation, value mixing, cache append), one launch; returns
+    the queries. See the reference."""
+    if src.is_cuda:
+        q = torch.empty(src.shape[0], nq * d, dtype=src.dtype,
+                        device=src.device)
+        _native().qkv_rope_append(src, col0, nq, nkv, d, dv, bias, conv_w,
+                                  conv_state, rot_freq, half, vf, lam, q,
+                                  kcache, vcache, pos, lens, slots, T)
+        return q
+    return ref.qkv_rope_append(src, col0, nq, nkv, d, dv, kcache, vcache, pos,
+                               T, lens, slots, bias, conv_w, conv_state,
+                               rot_freq, half, vf, lam)
+
+
+def scan_tiles(d: int, dv: int) -> int:
+    """Column tiles of the matrix memory's scan (each keeps its own copy of
+    the normalizer and the running maximum)."""
+    return -(-dv // (64 if d <= 256 else 32))
+
+
+def gla_scan(src, q0: int, k0: int, v0: int, a0: int, a2t, ab, inv_tau: float,
+             qscale: float, state, pos, T: int, lens=None,
+             slots=None) -> torch.Tensor:
+    """Linear attention with a low-rank decay per key channel (fp32)."""
+    if src.is_cuda:
+        # padded rows of a ragged batch are never written by the kernel
+        o = (torch.zeros if lens is not None else torch.empty)(
+            src.shape[0], state.shape[1] * state.shape[3],
+            dtype=torch.float32, device=src.device)
+        _native().gla_scan(src, q0, k0, v0, a0, a2t, ab, inv_tau, qscale,
+                           state, o, pos, lens, slots, T)
+        return o
+    return ref.gla_scan(src, q0, k0, v0, a0, a2t, ab, inv_tau, qscale, state,
+                        pos, T, lens, slots)
+
+
+def mlstm_scan(src, q0: int, k0: int, v0: int, i0: int, f0: int, ib, fb,
+               cap: float, qscale: float, state, nst, mst, pos, T: int,
+               lens=None, slots=None) -> torch.Tensor:
+    """Matrix memory with exponential gates and a running maximum (fp32)."""
+    if src.is_cuda:
+        o = (torch.zeros if lens is not None else torch.empty)(
+            src.shape[0], state.shape[1] * state.shape[3],
+            dtype=torch.float32, device=src.device)
+        _native().mlstm_scan(src, q0, k0, v0, i0, f0, ib, fb, cap, qscale,
+                             state, nst, mst, o, pos, lens, slots, T)
+        return o
+    return ref.mlstm_scan(src, q0, k0, v0, i0, f0, ib, fb, cap, qscale, state,
+                          nst, mst, pos, T, lens, slots)

@@ -17,6 +17,14 @@
 // (block means written by kv_pool_update) for every c < (i - window + 1) /
 // pool, in the same softmax and without a distance penalty.
 //
+// Kept first tokens (keep > 0, with a window): beside the window every query
+// sees the keys j < keep (at their true positions), in the same softmax. Tiles
+// between the kept keys and the window are not visited.
+//
+// Output gate (gate given): head h's result is multiplied by gate_scale *
+// sigmoid(gate[row, gate_col + h]) before it is rounded; the rows of the output
+// may be a column range of a wider buffer (row stride out_ld).
+//
 // Chunked visibility (chunk > 0): a query sees key j only inside its own block
 // of `chunk` positions, j >= (i / chunk) * chunk, blocks counted from position
 // 0. Sigmoid weights (sbias given): no softmax; a visible key weighs
@@ -117,6 +125,13 @@ struct ModParams {
   // value pointer is the key pointer and VS = D.
   int VS, vshare;
   float scale, softcap;
+  int keep;            // first keys that stay visible beside the window
+  int64_t out_ld;      // elements between consecutive output rows
+  // per-head output gate: columns gate_col.. of gate rows (same dtype), or null
+  const void* gate;
+  int64_t gate_ld;
+  int gate_col;
+  float gate_scale;
 };
 
 // pooled entries visible to a query at position i
@@ -140,6 +155,15 @@ template <bool FAST> __device__ __forceinline__ float m_sigmoid(float x) {
 }
 template <bool FAST> __device__ __forceinline__ float m_log1p(float x) {
   return FAST ? __logf(1.f + x) : log1pf(x);
+}
+
+// factor of head h's result in output row `row`
+template <typename T>
+__device__ __forceinline__ float out_gate(const ModParams& P, int64_t row, int h) {
+  if (P.gate == nullptr) return 1.f;
+  const float g =
+      ldv<T>(reinterpret_cast<const T*>(P.gate) + row * P.gate_ld + P.gate_col + h);
+  return P.gate_scale / (1.f + expf(-g));
 }
 
 // 16 B global -> LDS row copies (rows are 8 B aligned for bf16, 4 B for fp32)
@@ -240,14 +264,21 @@ __global__ __launch_bounds__(256) void attn_mod_rows(
   const int np_max = pool_count(p0 + t0 + nt - 1, P.window, P.pool, P.Sp);
   const int n_pc = (np_max + kChunkR - 1) / kChunkR;
   const int tok0 = kv_begin & ~(kChunkR - 1);
+  // kept first tokens in chunks of their own, as far as the range misses them
+  const int keep_end = min(P.keep, tok0);
+  const int n_kc = (keep_end + kChunkR - 1) / kChunkR;
   const int n_tc = kv_end > tok0 ? (kv_end - tok0 + kChunkR - 1) / kChunkR : 0;
   const int64_t pkbase = ((int64_t)slot * P.Hkv + hkv) * P.Sp * D;
   const int64_t pvbase = ((int64_t)slot * P.Hkv + hkv) * P.Sp * DV;
 
-  for (int c = split; c < n_pc + n_tc; c += splits) {
+  for (int c = split; c < n_pc + n_kc + n_tc; c += splits) {
     const bool pooled = c < n_pc;
-    const int s0 = pooled ? c * kChunkR : tok0 + (c - n_pc) * kChunkR;
-    const int valid = min(kChunkR, (pooled ? np_max : kv_end) - s0);
+    const bool kept = !pooled && c < n_pc + n_kc;
+    const int s0 = pooled ? c * kChunkR
+                   : kept ? (c - n_pc) * kChunkR
+                          : tok0 + (c - n_pc - n_kc) * kChunkR;
+    const int valid =
+        min(kChunkR, (pooled ? np_max : kept ? keep_end : kv_end) - s0);
     const T* kc = pooled ? reinterpret_cast<const T*>(P.pk) + pkbase
                          : kc_tok + kbase;
     const T* vc = pooled ? reinterpret_cast<const T*>(P.pv) + pvbase
@@ -289,7 +320,8 @@ __global__ __launch_bounds__(256) void attn_mod_rows(
       const int r = wid + 4 * rr;
       const int j = s0 + lane;
       bool live = lane < valid && j < lim;
-      if (!pooled && P.window > 0) live = live && (j > i - P.window);
+      if (!pooled && P.window > 0)
+        live = live && (j > i - P.window || j < P.keep);
       if (P.chunk > 0) live = live && (j >= cb[rr]);
       float s = dot_lds(&k_lds[lane * PK], &q_lds[r * PK], D) * tmp[rr];
       if (cap > 0.f) s = cap * m_tanh<FAST>(s * inv_cap);
@@ -381,8 +413,10 @@ __global__ __launch_bounds__(256) void attn_mod_rows(
       c = m_exp<FAST>(m[rr] - m2);
       l[rr] = l[rr] * c + m_exp<FAST>(sk - m2);
     }
-    const float inv = sig ? 1.f : (l[rr] > 0.f ? c / l[rr] : 0.f);
-    T* op = out + ((int64_t)b * P.T + t) * P.Hq * DV + (int64_t)h * DV;
+    const int64_t orow = (int64_t)b * P.T + t;
+    const float inv = (sig ? 1.f : (l[rr] > 0.f ? c / l[rr] : 0.f)) *
+                      out_gate<T>(P, orow, h);
+    T* op = out + orow * P.out_ld + (int64_t)h * DV;
 #pragma unroll
     for (int jj = 0; jj < 4; ++jj) {
       if (PAIR) {
@@ -399,17 +433,20 @@ __global__ __launch_bounds__(256) void attn_mod_rows(
 // merge the splits of one (batch row, head): one wave per output row
 template <typename T>
 __global__ __launch_bounds__(64) void attn_mod_combine(
-    const float* __restrict__ partial, T* __restrict__ out,
-    const float* __restrict__ sinks, const int* __restrict__ pos,
-    const int* __restrict__ slots, const int Hq, const int DV,
-    const int splits, const int Bc, const int plain_sum) {
+    const float* __restrict__ partial, T* __restrict__ out, const int splits,
+    const int plain_sum, const ModParams P) {
+  const int Hq = P.Hq, DV = P.DV;
   const int b = blockIdx.x / Hq, h = blockIdx.x % Hq;
+  if (P.lens && P.lens[b] <= 0) return;      // idle row: no partials
+  const float* sinks = P.sinks;
   const float* pp = partial + (int64_t)blockIdx.x * splits * (DV + 2);
+  const float gate = out_gate<T>(P, b, h);
+  T* op = out + b * P.out_ld + (int64_t)h * DV;
   if (plain_sum) {             // unnormalized weights: the splits just add
     for (int dv = threadIdx.x; dv < DV; dv += 64) {
       float a = 0.f;
       for (int s = 0; s < splits; ++s) a += pp[s * (DV + 2) + dv];
-      stv<T>(out + (int64_t)blockIdx.x * DV + dv, a);
+      stv<T>(op + dv, a * gate);
     }
     return;
   }
@@ -419,12 +456,12 @@ __global__ __launch_bounds__(64) void attn_mod_combine(
   float L = sinks ? expf(sinks[h] - M) : 0.f;
   for (int s = 0; s < splits; ++s)
     L += pp[s * (DV + 2) + DV + 1] * expf(pp[s * (DV + 2) + DV] - M);
-  const float inv = L > 0.f ? 1.f / L : 0.f;
+  const float inv = (L > 0.f ? 1.f / L : 0.f) * gate;
   for (int dv = threadIdx.x; dv < DV; dv += 64) {
     float a = 0.f;
     for (int s = 0; s < splits; ++s)
       a += pp[s * (DV + 2) + dv] * expf(pp[s * (DV + 2) + DV] - M);
-    stv<T>(out + (int64_t)blockIdx.x * DV + dv, a * inv);
+    stv<T>(op + dv, a * inv);
   }
 }
 
@@ -499,17 +536,19 @@ __global__ __launch_bounds__(256) void attn_mod_mfma(
   const short* kp_tok = kp;
   const short* vp_tok = vp;
 
-  // phase 0: pooled entries (block means before the window); phase 1: tokens
-  for (int ph = P.pool > 0 ? 0 : 1; ph < 2; ++ph) {
+  // phase 0: pooled entries (block means before the window); phase 1: kept
+  // first tokens that the token range misses; phase 2: the token range
+  int tok0 = 0;
+  if (P.window > 0) tok0 = max(0, p0 + tile0 - P.window + 1) & ~(ST - 1);
+  if (P.chunk > 0)
+    tok0 = max(tok0, (((p0 + tile0) / P.chunk) * P.chunk) & ~(ST - 1));
+  for (int ph = P.pool > 0 ? 0 : (P.keep > 0 ? 1 : 2); ph < 3; ++ph) {
   const bool pooled = ph == 0;
   const int Sdim = pooled ? P.Sp : P.Smax;
   const int s_end = pooled ? pool_count(p0 + q_hi, P.window, P.pool, P.Sp)
-                           : min(P.Smax, p0 + q_hi + 1);
-  int s_begin = 0;
-  if (!pooled && P.window > 0)
-    s_begin = max(0, p0 + tile0 - P.window + 1) & ~(ST - 1);
-  if (!pooled && P.chunk > 0)
-    s_begin = max(s_begin, (((p0 + tile0) / P.chunk) * P.chunk) & ~(ST - 1));
+                    : ph == 1 ? min(P.keep, tok0)
+                              : min(P.Smax, p0 + q_hi + 1);
+  const int s_begin = ph == 2 ? tok0 : 0;
   kp = pooled ? reinterpret_cast<const short*>(P.pk) +
                     ((int64_t)slot * P.Hkv + hk) * P.Sp * D
               : kp_tok;
@@ -564,7 +603,7 @@ __global__ __launch_bounds__(256) void attn_mod_mfma(
         } else {
           if (P.r1) val -= r1 * __logf(1.f + r2 * (float)max(i - j, 0));
           dead = (j > i) || (qq >= n) || (j >= P.Smax);
-          if (P.window > 0) dead |= (j <= i - P.window);
+          if (P.window > 0) dead |= (j <= i - P.window && j >= P.keep);
           if (P.chunk > 0) dead |= (j < (i / P.chunk) * P.chunk);
         }
         if (sig)
@@ -626,8 +665,10 @@ __global__ __launch_bounds__(256) void attn_mod_mfma(
       c = __expf(m_run[r] - m2);
       l_run[r] = l_run[r] * c + __expf(sk - m2);
     }
-    const float inv = sig ? 1.f : (l_run[r] > 0.f ? c / l_run[r] : 0.f);
-    short* op = out + ((int64_t)b * P.T + qq) * P.Hq * DV + (int64_t)h * DV;
+    const int64_t orow = (int64_t)b * P.T + qq;
+    const float inv = (sig ? 1.f : (l_run[r] > 0.f ? c / l_run[r] : 0.f)) *
+                      out_gate<short>(P, orow, h);
+    short* op = out + orow * P.out_ld + (int64_t)h * DV;
 #pragma unroll
     for (int nn = 0; nn < NV; ++nn) {
       const int dv = nn * 16 + row;
@@ -703,7 +744,13 @@ __global__ __launch_bounds__(256) void attn_mod_mfma_heads(
 
   const int s_end = min(P.Smax, i + 1);
   const int s_begin = P.window > 0 ? (max(0, i - P.window + 1) & ~(ST - 1)) : 0;
-  const int tiles = s_end > s_begin ? (s_end - s_begin + ST - 1) / ST : 0;
+  // tiles of kept first tokens come first, as far as the range misses them
+  const int kt = (min(P.keep, s_begin) + ST - 1) / ST;
+  const int tiles =
+      kt + (s_end > s_begin ? (s_end - s_begin + ST - 1) / ST : 0);
+  auto tile_at = [&](const int tile) {
+    return tile < kt ? tile * ST : s_begin + (tile - kt) * ST;
+  };
 
   // the next tile's key rows travel from memory into registers while the
   // current tile is worked on
@@ -722,10 +769,10 @@ __global__ __launch_bounds__(256) void attn_mod_mfma_heads(
       kreg[v] = z;
     }
   };
-  if (split < tiles) load_tile(s_begin + split * ST);
+  if (split < tiles) load_tile(tile_at(split));
 
   for (int tile = split; tile < tiles; tile += splits) {
-    const int s0 = s_begin + tile * ST;
+    const int s0 = tile_at(tile);
     __syncthreads();
 #pragma unroll
     for (int v = 0; v < KV; ++v) {
@@ -733,7 +780,7 @@ __global__ __launch_bounds__(256) void attn_mod_mfma_heads(
       const int sr = idx / (DP / 8), dc = (idx % (DP / 8)) * 8;
       *reinterpret_cast<short8*>(&k_lds[sr * KP + dc]) = kreg[v];
     }
-    if (tile + splits < tiles) load_tile(s0 + splits * ST);
+    if (tile + splits < tiles) load_tile(tile_at(tile + splits));
     if (P.vshare) {
       // the staged key rows are the values: transpose them inside LDS, the
       // 32 keys of a value dimension across neighbouring lanes (consecutive
@@ -779,7 +826,7 @@ __global__ __launch_bounds__(256) void attn_mod_mfma_heads(
         if (cap > 0.f) val = cap * fast_tanh(val * inv_cap);
         if (P.r1) val -= r1[r] * __logf(1.f + r2[r] * (float)max(i - j, 0));
         bool dead = (j > i) || (j >= P.Smax) || !alive[r];
-        if (P.window > 0) dead |= (j <= i - P.window);
+        if (P.window > 0) dead |= (j <= i - P.window && j >= P.keep);
         p_val[sub][r] = dead ? -INFINITY : val;
       }
     }
@@ -869,7 +916,9 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
               c10::optional<torch::Tensor> pool_k,
               c10::optional<torch::Tensor> pool_v, int64_t pool,
               int64_t v_dim, int64_t chunk,
-              c10::optional<torch::Tensor> sig_bias) {
+              c10::optional<torch::Tensor> sig_bias, int64_t keep,
+              c10::optional<torch::Tensor> gate, int64_t gate_col,
+              double gate_scale) {
   // no value cache: values = the first v_dim entries of the key rows
   const bool vshare = !vcache_opt.has_value();
   const torch::Tensor& vcache = vshare ? kcache : *vcache_opt;
@@ -889,8 +938,10 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
              "q [B*T, Hq*D]");
   const int Hq = q.size(1) / D;
   DNET_CHECK(Hq % Hkv == 0, "grouped heads");
-  DNET_CHECK(out.is_contiguous() && out.size(0) == M &&
-                 out.size(1) == (int64_t)Hq * DV, "out [B*T, Hq*DV]");
+  DNET_CHECK(out.dim() == 2 && out.size(0) == M &&
+                 out.size(1) == (int64_t)Hq * DV && out.stride(1) == 1 &&
+                 (M <= 1 || out.stride(0) >= out.size(1)),
+             "out [B*T, Hq*DV], rows may be a column range");
   DNET_CHECK(q.scalar_type() == kcache.scalar_type() &&
                  q.scalar_type() == vcache.scalar_type() &&
                  q.scalar_type() == out.scalar_type(), "dtypes");
@@ -916,6 +967,20 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
   P.D = D; P.DV = DV; P.window = (int)window;
   P.VS = vshare ? D : DV; P.vshare = vshare ? 1 : 0;
   P.scale = (float)scale; P.softcap = (float)softcap;
+  DNET_CHECK(keep == 0 || (window > 0 && keep > 0 && pool == 0 && chunk <= 0),
+             "kept first tokens come with a window");
+  P.keep = (int)keep;
+  P.out_ld = out.stride(0);
+  P.gate = nullptr;
+  P.gate_ld = 0; P.gate_col = 0; P.gate_scale = (float)gate_scale;
+  if (gate.has_value()) {
+    DNET_CHECK(gate->dim() == 2 && gate->is_contiguous() && gate->size(0) == M &&
+                   gate->scalar_type() == q.scalar_type() && gate_col >= 0 &&
+                   gate_col + Hq <= gate->size(1), "gate columns [B*T, Hq]");
+    P.gate = gate->data_ptr();
+    P.gate_ld = gate->size(1);
+    P.gate_col = (int)gate_col;
+  }
   P.pk = P.pv = nullptr;
   P.pool = 0; P.Sp = 0;
   if (pool > 0) {
@@ -981,8 +1046,8 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
 #undef AH_V
 #undef AH
     hipLaunchKernelGGL((attn_mod_combine<short>), dim3((unsigned)(B * Hq)),
-                       dim3(64), 0, stream, part, (short*)out.data_ptr(),
-                       P.sinks, P.pos, P.slots, Hq, DV, ns, Bc, 0);
+                       dim3(64), 0, stream, part, (short*)out.data_ptr(), ns,
+                       0, P);
     return;
   }
   // bf16 prompts: matrix-core kernel (head sizes padded to its tile classes)
@@ -1037,8 +1102,7 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
     if (ns > 1)                                                             \
       hipLaunchKernelGGL((attn_mod_combine<TT>), dim3((unsigned)(B * Hq)),  \
                          dim3(64), 0, stream, part, (TT*)out.data_ptr(),    \
-                         P.sinks, P.pos, P.slots, Hq, DV, ns, Bc,           \
-                         sig ? 1 : 0);                                      \
+                         ns, sig ? 1 : 0, P);                               \
   } while (0)
   if (f32) {
     if (vec) AR(float, true); else AR(float, false);

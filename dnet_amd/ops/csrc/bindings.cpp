@@ -95,8 +95,6 @@ void gated_group_rmsnorm(torch::Tensor y, torch::Tensor gate_src,
 void act_slice(torch::Tensor x, int64_t col0, torch::Tensor y, int64_t kind);
 void gelu_gather_mul(torch::Tensor z, torch::Tensor table,
                      torch::Tensor tokens, int64_t col0, torch::Tensor y);
-void clamped_glu(torch::Tensor gu, torch::Tensor y, double alpha,
-                 double limit);
 void kv_pool_update(torch::Tensor kcache, torch::Tensor vcache,
                     torch::Tensor pool_k, torch::Tensor pool_v,
                     torch::Tensor pos, c10::optional<torch::Tensor> lens,
@@ -130,7 +128,30 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
               c10::optional<torch::Tensor> pool_k,
               c10::optional<torch::Tensor> pool_v, int64_t pool,
               int64_t v_dim, int64_t chunk,
-              c10::optional<torch::Tensor> sig_bias);
+              c10::optional<torch::Tensor> sig_bias, int64_t keep,
+              c10::optional<torch::Tensor> gate, int64_t gate_col,
+              double gate_scale);
+void qkv_rope_append(torch::Tensor src, int64_t col0, int64_t nq, int64_t nkv,
+                     int64_t d, int64_t dv, c10::optional<torch::Tensor> bias,
+                     c10::optional<torch::Tensor> conv_w,
+                     c10::optional<torch::Tensor> conv_state,
+                     c10::optional<torch::Tensor> rot_freq, bool half,
+                     c10::optional<torch::Tensor> vf,
+                     c10::optional<torch::Tensor> lam, torch::Tensor q,
+                     torch::Tensor kcache, torch::Tensor vcache,
+                     torch::Tensor pos, c10::optional<torch::Tensor> lens,
+                     c10::optional<torch::Tensor> slots, int64_t T);
+void gla_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0, int64_t a0,
+              torch::Tensor a2t, torch::Tensor ab, double inv_tau,
+              double qscale, torch::Tensor state, torch::Tensor o,
+              torch::Tensor pos, c10::optional<torch::Tensor> lens,
+              c10::optional<torch::Tensor> slots, int64_t T);
+void mlstm_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0,
+                int64_t i0, int64_t f0, torch::Tensor ib, torch::Tensor fb,
+                double cap, double qscale, torch::Tensor state,
+                torch::Tensor nst, torch::Tensor mst, torch::Tensor o,
+                torch::Tensor pos, c10::optional<torch::Tensor> lens,
+                c10::optional<torch::Tensor> slots, int64_t T);
 void pair_hash_embed(torch::Tensor tokens, torch::Tensor embed,
                      torch::Tensor table, torch::Tensor prev,
                      torch::Tensor out, torch::Tensor pos,
@@ -198,11 +219,15 @@ void cache_append(torch::Tensor src, int64_t col0, torch::Tensor cache,
                   torch::Tensor pos, c10::optional<torch::Tensor> lens,
                   c10::optional<torch::Tensor> slots, int64_t T);
 void gated_act(torch::Tensor gu, c10::optional<torch::Tensor> scale,
-               torch::Tensor y, int64_t kind);
+               torch::Tensor y, int64_t kind, double alpha, double limit);
 void moe_router(c10::optional<torch::Tensor> x, torch::Tensor w,
                 c10::optional<torch::Tensor> logits, torch::Tensor idx,
                 torch::Tensor val, torch::Tensor we,
-                c10::optional<torch::Tensor> gate);
+                c10::optional<torch::Tensor> gate,
+                c10::optional<torch::Tensor> corr, int64_t groups,
+                int64_t keep, double scale);
+void moe_clamped_rows(torch::Tensor x, torch::Tensor w, torch::Tensor we,
+                      torch::Tensor act, double alpha, double limit);
 void moe_plan(torch::Tensor idx, torch::Tensor order, torch::Tensor at,
               torch::Tensor counts);
 void moe_gather(torch::Tensor x, torch::Tensor order, torch::Tensor val,
@@ -288,7 +313,6 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "unary activation of a column range (relu^2, tanh)");
   m.def("gelu_gather_mul", &dnet::gelu_gather_mul,
         "gelu_tanh(z) * table[token, col0:col0+n]");
-  m.def("clamped_glu", &dnet::clamped_glu, "clamped GLU of [gate | up]");
   m.def("kv_pool_update", &dnet::kv_pool_update,
         "block means of the KV cache for the blocks a step completes");
   m.def("causal_conv_silu", &dnet::causal_conv_silu,
@@ -329,9 +353,21 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("cache_append", &dnet::cache_append,
         "projection columns as they are into cache rows");
   m.def("gated_act", &dnet::gated_act,
-        "act(s gate) * (s up), silu or tanh-gelu, optional row factor");
+        "act(s gate) * (s up), silu or tanh-gelu, or the clamped gated unit, "
+        "optional row factor");
+  m.def("qkv_rope_append", &dnet::qkv_rope_append,
+        "q/k/v columns: bias or short convolution, rotation, value mixing, "
+        "cache append");
+  m.def("gla_scan", &dnet::gla_scan,
+        "linear attention with a low-rank decay per key channel");
+  m.def("mlstm_scan", &dnet::mlstm_scan,
+        "matrix memory with exponential gates and a running maximum");
+  m.def("moe_clamped_rows", &dnet::moe_clamped_rows,
+        "clamped gated experts on a decode batch, routing weight on the "
+        "result (matrix cores)");
   m.def("moe_router", &dnet::moe_router,
-        "sigmoid router: top-k scores kept as they are, shared-expert gate");
+        "sigmoid router: top-k scores times a constant, optional correction, "
+        "expert groups and shared-expert gate");
   m.def("moe_plan", &dnet::moe_plan, "routed entries sorted by expert");
   m.def("moe_gather", &dnet::moe_gather, "rows and scales of sorted entries");
   m.def("moe_gateup_rows", &dnet::moe_gateup_rows,

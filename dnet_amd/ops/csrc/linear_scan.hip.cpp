@@ -1,0 +1,383 @@
+// Linear-attention recurrences with input-dependent gates (gfx950), fp32 state
+// per slot and head:
+//
+//   gla_scan    S <- diag(alpha_t) S + k v^T ; o = S^T q, a decay per key
+//               channel alpha = sigmoid(A2 a1 + b)^(1/tau) (low-rank A2 a1)
+//   mlstm_scan  matrix memory with exponential gates and a running maximum m:
+//               m' = max(f + m, i); S <- e^(f+m-m') S + e^(i-m') k v^T, n like
+//               S with k alone; o = S^T q / (max(|n . q|, e^-m') + 1e-6);
+//               i = cap tanh(./cap), f = logsigmoid(cap tanh(./cap))
+//
+// Geometry is the cache's: token (b,t) = row b*T+t sits at position pos[b]+t of
+// slot slots[b] (default b); tokens t >= lens[b] are padding. State is taken as
+// zero at position 0 and written only by rows with real tokens. Gates, decays,
+// states and results are fp32 whatever the activation dtype ("short" stands
+// for bf16 bits).
+//
+// Layout: a workgroup owns a tile of JB value columns of one head of one batch
+// row and walks the tokens in order; thread (column j, slice s) keeps rows
+// [R s, R s + R) of column j in registers, the slices of a column are
+// neighbouring lanes. Tokens are staged through LDS in chunks, with every
+// gate evaluated once per chunk; the chunk's results are gathered in LDS and
+// written out as rows. The matrix memory's normalizer n is one more column
+// (of ones) on a wave of its own, which also forms the gates and the running
+// maximum; every column tile keeps its own copy of n and m, so that no
+// workgroup reads what another one writes.
+#include "common.h"
+
+namespace dnet {
+
+namespace {
+
+template <typename T> __device__ __forceinline__ float ldx(const T* p);
+template <> __device__ __forceinline__ float ldx<float>(const float* p) { return *p; }
+template <> __device__ __forceinline__ float ldx<short>(const short* p) { return bits2f(*p); }
+
+bool is_bf16(const torch::Tensor& t) { return t.scalar_type() == torch::kBFloat16; }
+bool is_f32(const torch::Tensor& t) { return t.scalar_type() == torch::kFloat32; }
+
+__device__ __forceinline__ float log_sigmoid(float z) {
+  return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+}
+
+constexpr int kGla = 0, kMlstm = 1;
+constexpr float kDenEps = 1e-6f;
+
+struct ScanArgs {
+  const void* src;           // projection rows [B*T, ld]
+  float* state;              // [Bc, H, d, dv]
+  float* o;                  // [B*T, H*dv]
+  const int* pos;
+  const int* lens;
+  const int* slots;
+  // gla: low-rank input at column a0, a2t [rank][H*d], bias [H*d]
+  const float* a2t;
+  const float* ab;
+  // mlstm: gate columns i0, f0 with biases, n [Bc, H, NT, d], m [Bc, H, NT]
+  const float* ib;
+  const float* fb;
+  float* nst;
+  float* mst;
+  int64_t ld;
+  int q0, k0, v0, a0, rank, i0, f0, T, Bc, H, d, dv, JB, NS, TC, NT;
+  float qscale, inv_tau, cap;
+};
+
+template <typename T, int R, int KIND>
+__global__ __launch_bounds__(1024) void linear_scan_kernel(const ScanArgs a) {
+  const int h = blockIdx.x / a.NT, tile = blockIdx.x % a.NT, b = blockIdx.y;
+  const int n = a.lens ? min(a.lens[b], a.T) : a.T;
+  const int slot = a.slots ? a.slots[b] : b;
+  const int p0 = a.pos[b];
+  if (n <= 0 || slot < 0 || slot >= a.Bc || p0 < 0) return;   // uniform
+  const int d = a.d, dv = a.dv, JB = a.JB, NS = a.NS, TC = a.TC;
+  const int j0 = tile * JB;
+  const int DR = NS * R;                    // key rows incl. padding
+  const int DP = NS * (R + 4);              // LDS pitch of one token: slices
+                                            // four banks apart
+  const int JP = JB + 1;                    // columns and the normalizer's
+  const int nmain = JB * NS, lane = threadIdx.x & 63;
+  const bool ncol = KIND == kMlstm && (int)threadIdx.x >= nmain;  // wave-uniform
+  const int jl = ncol ? JB : threadIdx.x / NS;
+  const int sl = ncol ? lane % NS : threadIdx.x % NS;
+  const int j = j0 + jl;
+  const bool col_ok = !ncol && j < dv;
+
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  float* sQ = sm;                           // [TC][DP]
+  float* sK = sQ + TC * DP;
+  float* sA = sK + TC * DP;                 // gla: decays
+  float* sV = sA + (KIND == kGla ? TC * DP : 0);   // [TC][JP]
+  float* sO = sV + TC * JP;                 // [TC][JP]
+  float* sKeep = sO + TC * JP;              // mlstm: [TC] each; gla: [TC][rank]
+  float* sPut = sKeep + TC;
+  float* sEm = sPut + TC;
+  float* sZ = sKeep;
+
+  float S[R];
+  float* sp = a.state + (((int64_t)slot * a.H + h) * d) * dv;
+  float* np = nullptr;
+  float* mp = nullptr;
+  float m = 0.f;
+  if constexpr (KIND == kMlstm) {
+    np = a.nst + (((int64_t)slot * a.H + h) * a.NT + tile) * d;
+    mp = a.mst + ((int64_t)slot * a.H + h) * a.NT + tile;
+    if (p0 > 0) m = *mp;
+  }
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int row = sl * R + r;
+    S[r] = 0.f;
+    if (p0 > 0 && row < d) {
+      if (ncol) S[r] = np[row];
+      else if (col_ok) S[r] = sp[(int64_t)row * dv + j];
+    }
+  }
+  const T* src = reinterpret_cast<const T*>(a.src) + (int64_t)b * a.T * a.ld;
+
+  for (int t0 = 0; t0 < n; t0 += TC) {
+    const int tc = min(TC, n - t0);
+    __syncthreads();                        // previous chunk consumed
+    if (ncol) {
+      float lf = 0.f, li = 0.f;
+      if (lane < tc) {
+        const T* sr = src + (int64_t)(t0 + lane) * a.ld;
+        const float iv = ldx<T>(sr + a.i0 + h) + a.ib[h];
+        const float fv = ldx<T>(sr + a.f0 + h) + a.fb[h];
+        li = a.cap * tanhf(iv / a.cap);
+        lf = log_sigmoid(a.cap * tanhf(fv / a.cap));
+      }
+      float before = 0.f, after = 0.f;
+      for (int t = 0; t < tc; ++t) {        // the running maximum, in order
+        const float f = __shfl(lf, t, 64), i = __shfl(li, t, 64);
+        const float mn = fmaxf(f + m, i);
+        if (lane == t) {
+          before = f + m;
+          after = mn;
+        }
+        m = mn;
+      }
+      if (lane < tc) {
+        sKeep[lane] = expf(before - after);
+        sPut[lane] = expf(li - after);
+        sEm[lane] = expf(-after);
+        sV[lane * JP + JB] = 1.f;
+      }
+    } else {
+      for (int idx = threadIdx.x; idx < tc * DR; idx += nmain) {
+        const int tt = idx / DR, i = idx % DR;
+        const T* sr = src + (int64_t)(t0 + tt) * a.ld + h * d + i;
+        const int at = tt * DP + (i / R) * (R + 4) + (i % R);
+        sQ[at] = i < d ? ldx<T>(sr + a.q0) * a.qscale : 0.f;
+        sK[at] = i < d ? ldx<T>(sr + a.k0) : 0.f;
+      }
+      for (int idx = threadIdx.x; idx < tc * JB; idx += nmain) {
+        const int tt = idx / JB, c = idx % JB;
+        sV[tt * JP + c] =
+            j0 + c < dv ? ldx<T>(src + (int64_t)(t0 + tt) * a.ld + a.v0 +
+                                 h * dv + j0 + c)
+                        : 0.f;
+      }
+      if constexpr (KIND == kGla)
+        for (int idx = threadIdx.x; idx < tc * a.rank; idx += nmain) {
+          const int tt = idx / a.rank, r = idx % a.rank;
+          sZ[idx] = ldx<T>(src + (int64_t)(t0 + tt) * a.ld + a.a0 + r);
+        }
+    }
+    __syncthreads();
+    if constexpr (KIND == kGla) {
+      // decays of four tokens per work item (a weight is read once for them)
+      const int groups = (tc + 3) / 4;
+      for (int idx = threadIdx.x; idx < DR * groups; idx += nmain) {
+        const int i = idx % DR, tg = (idx / DR) * 4;
+        float z[4] = {0.f, 0.f, 0.f, 0.f};
+        if (i < d) {
+          const float* wp = a.a2t + h * d + i;
+#pragma unroll
+          for (int u = 0; u < 4; ++u) z[u] = a.ab[h * d + i];
+#pragma unroll 4
+          for (int r = 0; r < a.rank; ++r) {
+            const float w = wp[(int64_t)r * a.H * d];
+#pragma unroll
+            for (int u = 0; u < 4; ++u)
+              z[u] = fmaf(w, sZ[min(tg + u, tc - 1) * a.rank + r], z[u]);
+          }
+        }
+        const int at = (i / R) * (R + 4) + (i % R);
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          if (tg + u < tc)
+            sA[(tg + u) * DP + at] =
+                i < d ? expf(log_sigmoid(z[u]) * a.inv_tau) : 0.f;
+      }
+      __syncthreads();
+    }
+    for (int tt = 0; tt < tc; ++tt) {
+      const int base = tt * DP + sl * (R + 4);
+      const float4* kp = reinterpret_cast<const float4*>(sK + base);
+      const float4* qp = reinterpret_cast<const float4*>(sQ + base);
+      float vj = sV[tt * JP + jl], acc = 0.f;
+      if constexpr (KIND == kGla) {
+        const float4* ap = reinterpret_cast<const float4*>(sA + base);
+#pragma unroll
+        for (int r4 = 0; r4 < R / 4; ++r4) {
+          const float4 kv = kp[r4], qv = qp[r4], av = ap[r4];
+          S[4 * r4 + 0] = fmaf(kv.x, vj, av.x * S[4 * r4 + 0]);
+          S[4 * r4 + 1] = fmaf(kv.y, vj, av.y * S[4 * r4 + 1]);
+          S[4 * r4 + 2] = fmaf(kv.z, vj, av.z * S[4 * r4 + 2]);
+          S[4 * r4 + 3] = fmaf(kv.w, vj, av.w * S[4 * r4 + 3]);
+          acc = fmaf(S[4 * r4 + 0], qv.x, acc);
+          acc = fmaf(S[4 * r4 + 1], qv.y, acc);
+          acc = fmaf(S[4 * r4 + 2], qv.z, acc);
+          acc = fmaf(S[4 * r4 + 3], qv.w, acc);
+        }
+      } else {
+        const float keep = sKeep[tt];
+        vj *= sPut[tt];
+#pragma unroll
+        for (int r4 = 0; r4 < R / 4; ++r4) {
+          const float4 kv = kp[r4], qv = qp[r4];
+          S[4 * r4 + 0] = fmaf(kv.x, vj, keep * S[4 * r4 + 0]);
+          S[4 * r4 + 1] = fmaf(kv.y, vj, keep * S[4 * r4 + 1]);
+          S[4 * r4 + 2] = fmaf(kv.z, vj, keep * S[4 * r4 + 2]);
+          S[4 * r4 + 3] = fmaf(kv.w, vj, keep * S[4 * r4 + 3]);
+          acc = fmaf(S[4 * r4 + 0], qv.x, acc);
+          acc = fmaf(S[4 * r4 + 1], qv.y, acc);
+          acc = fmaf(S[4 * r4 + 2], qv.z, acc);
+          acc = fmaf(S[4 * r4 + 3], qv.w, acc);
+        }
+      }
+      for (int off = NS >> 1; off > 0; off >>= 1)
+        acc += __shfl_xor(acc, off, 64);
+      if (sl == 0) sO[tt * JP + jl] = acc;
+    }
+    __syncthreads();
+    for (int idx = threadIdx.x; idx < tc * JB; idx += blockDim.x) {
+      const int tt = idx / JB, c = idx % JB;
+      if (j0 + c >= dv) continue;
+      float v = sO[tt * JP + c];
+      if constexpr (KIND == kMlstm)
+        v /= fmaxf(fabsf(sO[tt * JP + JB]), sEm[tt]) + kDenEps;
+      a.o[((int64_t)b * a.T + t0 + tt) * (int64_t)a.H * dv + h * dv + j0 + c] = v;
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int row = sl * R + r;
+    if (row >= d) continue;
+    if (ncol) {
+      if (lane < NS) np[row] = S[r];
+    } else if (col_ok) {
+      sp[(int64_t)row * dv + j] = S[r];
+    }
+  }
+  if (ncol && lane == 0) *mp = m;
+}
+
+const int* idx32(const torch::Tensor& t, int64_t n) {
+  DNET_CHECK(t.scalar_type() == torch::kInt32 && t.is_contiguous() &&
+                 t.numel() >= n, "int32 index tensor [B]");
+  return t.data_ptr<int>();
+}
+
+const float* f32p(const torch::Tensor& t, int64_t n, const char* what) {
+  DNET_CHECK(is_f32(t) && t.is_contiguous() && t.numel() == n, what);
+  return t.data_ptr<float>();
+}
+
+// shared part of the two entry points: checks, geometry, launch shape
+void scan_launch(ScanArgs& a, int kind, const torch::Tensor& src, int64_t q0,
+                 int64_t k0, int64_t v0, double qscale, torch::Tensor& state,
+                 torch::Tensor& o, const torch::Tensor& pos,
+                 const c10::optional<torch::Tensor>& lens,
+                 const c10::optional<torch::Tensor>& slots, int64_t T,
+                 int64_t NT) {
+  const int64_t M = src.size(0), ld = src.size(1);
+  DNET_CHECK(src.dim() == 2 && src.is_contiguous() &&
+                 (is_bf16(src) || is_f32(src)), "src [B*T, ld]");
+  DNET_CHECK(T > 0 && M % T == 0, "rows = B*T");
+  const int64_t B = M / T;
+  DNET_CHECK(is_f32(state) && state.is_contiguous() && state.dim() == 4,
+             "state fp32 [Bc, H, d, dv]");
+  const int64_t H = state.size(1), d = state.size(2), dv = state.size(3);
+  DNET_CHECK(q0 >= 0 && k0 >= 0 && v0 >= 0 && q0 + H * d <= ld &&
+                 k0 + H * d <= ld && v0 + H * dv <= ld, "src columns");
+  DNET_CHECK(is_f32(o) && o.is_contiguous() && o.size(0) == M &&
+                 o.size(1) == H * dv, "o fp32 [B*T, H*dv]");
+  DNET_CHECK(d >= 1 && d <= 512 && dv >= 1, "1 <= head size <= 512");
+  if (!slots.has_value()) DNET_CHECK(B <= state.size(0), "more rows than slots");
+  if (M == 0) return;
+  a.src = src.data_ptr();
+  a.state = state.data_ptr<float>();
+  a.o = o.data_ptr<float>();
+  a.pos = idx32(pos, B);
+  a.lens = lens.has_value() ? idx32(*lens, B) : nullptr;
+  a.slots = slots.has_value() ? idx32(*slots, B) : nullptr;
+  a.ld = ld; a.q0 = (int)q0; a.k0 = (int)k0; a.v0 = (int)v0;
+  a.T = (int)T; a.Bc = (int)state.size(0); a.H = (int)H; a.d = (int)d;
+  a.dv = (int)dv; a.qscale = (float)qscale; a.NT = (int)NT;
+  const int R = d <= 32 ? 8 : (d <= 128 ? 16 : 32);
+  a.NS = 1;
+  while (a.NS * R < d) a.NS *= 2;           // power of two, <= 16
+  const int cols = (int)((dv + NT - 1) / NT);
+  const int unit = kWave / a.NS;            // whole waves
+  a.JB = (cols + unit - 1) / unit * unit;
+  const int threads = a.JB * a.NS + (kind == kMlstm ? kWave : 0);
+  DNET_CHECK(threads <= 1024, "column tiles too wide");
+  const int DP = a.NS * (R + 4);
+  auto floats = [&](int tc) {
+    return (size_t)tc * ((kind == kGla ? 3 : 2) * DP + 2 * (a.JB + 1) +
+                         (kind == kGla ? a.rank : 3));
+  };
+  a.TC = (int)std::min<int64_t>(16, T);
+  while (a.TC > 1 && floats(a.TC) * sizeof(float) > 56 * 1024) a.TC /= 2;
+  const size_t lds = floats(a.TC) * sizeof(float);
+  DNET_CHECK(lds <= 64 * 1024, "linear_scan: sizes exceed LDS");
+  const dim3 grid((unsigned)(H * NT), (unsigned)B);
+  auto st = current_stream();
+#define LS(TT, RR, KK)                                                        \
+  hipLaunchKernelGGL((linear_scan_kernel<TT, RR, KK>), grid, dim3(threads),   \
+                     lds, st, a)
+#define LS_R(TT, KK)                        \
+  do {                                      \
+    if (R == 8) LS(TT, 8, KK);              \
+    else if (R == 16) LS(TT, 16, KK);       \
+    else LS(TT, 32, KK);                    \
+  } while (0)
+#define LS_K(TT) do { if (kind == kGla) LS_R(TT, kGla); else LS_R(TT, kMlstm); } while (0)
+  if (is_bf16(src)) LS_K(short); else LS_K(float);
+#undef LS_K
+#undef LS_R
+#undef LS
+}
+
+}  // namespace
+
+void gla_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0, int64_t a0,
+              torch::Tensor a2t, torch::Tensor ab, double inv_tau,
+              double qscale, torch::Tensor state, torch::Tensor o,
+              torch::Tensor pos, c10::optional<torch::Tensor> lens,
+              c10::optional<torch::Tensor> slots, int64_t T) {
+  ScanArgs a = {};
+  const int64_t n = state.size(1) * state.size(2);
+  DNET_CHECK(a2t.dim() == 2 && a2t.size(1) == n, "a2t fp32 [rank, H*d]");
+  a.rank = (int)a2t.size(0);
+  DNET_CHECK(a.rank >= 1 && a.rank <= 2048 && a0 >= 0 &&
+                 a0 + a.rank <= src.size(1), "low-rank columns");
+  a.a2t = f32p(a2t, a.rank * n, "a2t fp32 [rank, H*d]");
+  a.ab = f32p(ab, n, "ab fp32 [H*d]");
+  a.a0 = (int)a0;
+  a.inv_tau = (float)inv_tau;
+  // column tiles of up to 64
+  const int64_t NT = (state.size(3) + 63) / 64;
+  scan_launch(a, kGla, src, q0, k0, v0, qscale, state, o, pos, lens, slots, T,
+              NT);
+}
+
+void mlstm_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0,
+                int64_t i0, int64_t f0, torch::Tensor ib, torch::Tensor fb,
+                double cap, double qscale, torch::Tensor state,
+                torch::Tensor nst, torch::Tensor mst, torch::Tensor o,
+                torch::Tensor pos, c10::optional<torch::Tensor> lens,
+                c10::optional<torch::Tensor> slots, int64_t T) {
+  ScanArgs a = {};
+  const int64_t Bc = state.size(0), H = state.size(1), d = state.size(2);
+  DNET_CHECK(nst.dim() == 4 && nst.size(0) == Bc && nst.size(1) == H &&
+                 nst.size(3) == d, "n fp32 [Bc, H, tiles, d]");
+  const int64_t NT = nst.size(2);
+  DNET_CHECK(NT >= 1 && (state.size(3) + NT - 1) / NT <= 64, "column tiles");
+  f32p(nst, Bc * H * NT * d, "n fp32 [Bc, H, tiles, d]");
+  f32p(mst, Bc * H * NT, "m fp32 [Bc, H, tiles]");
+  a.nst = nst.data_ptr<float>();
+  a.mst = mst.data_ptr<float>();
+  a.ib = f32p(ib, H, "gate bias fp32 [H]");
+  a.fb = f32p(fb, H, "gate bias fp32 [H]");
+  DNET_CHECK(i0 >= 0 && f0 >= 0 && i0 + H <= src.size(1) &&
+                 f0 + H <= src.size(1), "gate columns");
+  DNET_CHECK(cap > 0, "gate cap");
+  a.i0 = (int)i0; a.f0 = (int)f0; a.cap = (float)cap;
+  scan_launch(a, kMlstm, src, q0, k0, v0, qscale, state, o,
+              pos, lens, slots, T, NT);
+}
+
+}  // namespace dnet

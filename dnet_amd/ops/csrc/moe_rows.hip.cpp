@@ -1,13 +1,18 @@
-// Mixtures of experts whose routing weight scales the expert's INPUT (gfx950):
+// Mixtures of sigmoid-routed experts, the routing weight on an expert's input or
+// on its result (gfx950):
 //
-//   moe_router       fp32 sigmoid scores, the `top` largest kept as they are
-//                    (plus an optional shared-expert gate as the last row);
+//   moe_router       fp32 sigmoid scores, the `top` largest kept times a
+//                    constant (plus an optional shared-expert gate as the last
+//                    row), optionally chosen by score + correction inside the
+//                    best groups of neighbouring experts;
 //                    the products themselves are part of the kernel for few
 //                    rows, prompts hand in the logits of a library product
 //   moe_plan         entries (row, choice) sorted by expert, without host work
 //   moe_gather       the sorted entries' rows and scales
 //   moe_gateup_rows  every expert on every row of a decode batch, matrix
-//   moe_down_rows    cores (moe_up_rows: ungated experts, squared ReLU): an expert's weights are read once for all rows,
+//   moe_down_rows    cores (moe_up_rows: ungated experts, squared ReLU;
+//                    moe_clamped_rows: clamped gate, routing weight on the
+//                    result): an expert's weights are read once for all rows,
 //                    experts that no row chose are skipped on the device
 //   moe_merge        sum of each row's chosen results + gate * shared
 //
@@ -55,9 +60,14 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(
     const T* __restrict__ x, const float* __restrict__ w,
     const float* __restrict__ logits, int* __restrict__ idx,
     float* __restrict__ val, float* __restrict__ we, float* __restrict__ gate,
-    const int W, const int E, const int R, const int top) {
+    const float* __restrict__ corr, const int W, const int E, const int R,
+    const int top, const int groups, const int keep, const float scale) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  float* sc = sm;                                   // [R]
+  float* sc = sm;                                   // [R] logits, then choice
+  float* ss = sm + R;                               // [E] scores (biased choice)
+  float* gs = ss + E;                               // [groups]
+  // choice by score + correction and by groups; else by the logits
+  const bool biased = corr != nullptr || groups > 1;
   const int t = blockIdx.x;
   const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
   if (x != nullptr) {
@@ -106,13 +116,47 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(
   }
   __syncthreads();
   for (int e = threadIdx.x; e < R; e += blockDim.x) {
-    const float z = sc[e];
-    sc[e] = z > -1e30f ? z : -1e30f;        // (padding rows may hold NaN)
+    const float zr = sc[e];
+    const float z = zr > -1e30f ? zr : -1e30f;   // (padding rows may hold NaN)
+    sc[e] = z;
+    if (biased && e < E) {
+      const float s = 1.f / (1.f + expf(-z));
+      ss[e] = s;
+      sc[e] = corr ? s + corr[e] : s;
+    }
     if (e == E && gate) gate[t] = 1.f / (1.f + expf(-z));
     if (e < E) we[(int64_t)t * E + e] = 0.f;
   }
   __syncthreads();
   if (wid != 0) return;
+  if (groups > 1) {
+    // a group's score: the sum of its two largest choice scores; experts of
+    // all but the `keep` best groups (lower index first) drop out
+    const int gsz = E / groups;
+    for (int g = lane; g < groups; g += 64) {
+      float a = -1e37f, c = -1e37f;
+      for (int e = g * gsz; e < (g + 1) * gsz; ++e) {
+        const float s = sc[e];
+        if (s > a) {
+          c = a;
+          a = s;
+        } else if (s > c) {
+          c = s;
+        }
+      }
+      gs[g] = gsz > 1 ? a + c : a;
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // one wave only
+    for (int g = lane; g < groups; g += 64) {
+      const float s = gs[g];
+      int better = 0;
+      for (int o = 0; o < groups; ++o)
+        better += gs[o] > s || (gs[o] == s && o < g);
+      if (better >= keep)
+        for (int e = g * gsz; e < (g + 1) * gsz; ++e) sc[e] = -3e38f;
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  }
   for (int k = 0; k < top; ++k) {
     float bv = -2e38f;
     int bi = E;                             // chosen logits are set to -3e38
@@ -132,13 +176,13 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(
         bi = oi;
       }
     }
-    // top <= E: bi is always one of the experts
+    // top <= experts that can be chosen: bi is always one of them
     if (lane == 0) {
-      const float s = 1.f / (1.f + expf(-bv));
+      const float s = (biased ? ss[bi] : 1.f / (1.f + expf(-bv))) * scale;
       idx[(int64_t)t * top + k] = bi;
       val[(int64_t)t * top + k] = s;
       // never 0: a chosen expert must not look skipped to the row kernels
-      we[(int64_t)t * E + bi] = fmaxf(s, 1e-38f);
+      we[(int64_t)t * E + bi] = s != 0.f ? s : 1e-38f;
       sc[bi] = -3e38f;
     }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // one wave only
@@ -228,15 +272,17 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(
 // v_mfma_f32_16x16x32_bf16, the next group in flight while one is multiplied;
 // the partial sums fold wave by wave through LDS. GLU: the first half of the fragments are gate columns,
 // the second half the up columns beside them (8 NF columns of act), inputs
-// scaled by the routing weight; else 16 NF plain or squared-ReLU columns.
-constexpr int kPlain = 0, kGlu = 1, kReluSq = 2;
+// scaled by the routing weight (ClampGlu: clamped gate, the weight on the
+// result); else 16 NF plain or squared-ReLU columns.
+constexpr int kPlain = 0, kGlu = 1, kReluSq = 2, kClampGlu = 3;
 
 template <int MT, int NF, int NW, int U, int KIND>
 __global__ __launch_bounds__(NW * 64) void moe_rows_kernel(
     const short* __restrict__ x, const short* __restrict__ w,
     const float* __restrict__ we, short* __restrict__ out, const int K,
-    const int N, const int E, const int T, const int64_t x_expert) {
-  constexpr bool GLU = KIND == kGlu;
+    const int N, const int E, const int T, const int64_t x_expert,
+    const float alpha, const float limit) {
+  constexpr bool GLU = KIND == kGlu || KIND == kClampGlu;
   constexpr int NC = GLU ? NF / 2 : NF;      // column fragments of the result
   __shared__ f32x4 part[NW / 2][MT * NF][64];
   const int e = blockIdx.z;
@@ -374,7 +420,12 @@ __global__ __launch_bounds__(NW * 64) void moe_rows_kernel(
         const int t = m0 + m * 16 + hi * 4 + r;
         if (t >= T) continue;
         float v = acc[m][f][r];
-        if constexpr (GLU) {
+        if constexpr (KIND == kClampGlu) {
+          const float g = fminf(v, limit);
+          const float u = fminf(fmaxf(acc[m][NC + f][r], -limit), limit);
+          v = g * __builtin_amdgcn_rcpf(1.f + __expf(-alpha * g)) * (u + 1.f) *
+              we[(int64_t)t * E + e];
+        } else if constexpr (GLU) {
           const float s = we[(int64_t)t * E + e];
           const float g = v * s;
           v = g * __builtin_amdgcn_rcpf(1.f + __expf(-g)) *
@@ -441,7 +492,9 @@ __global__ __launch_bounds__(256) void moe_merge_kernel(
 void moe_router(c10::optional<torch::Tensor> x, torch::Tensor w,
                 c10::optional<torch::Tensor> logits, torch::Tensor idx,
                 torch::Tensor val, torch::Tensor we,
-                c10::optional<torch::Tensor> gate) {
+                c10::optional<torch::Tensor> gate,
+                c10::optional<torch::Tensor> corr, int64_t groups,
+                int64_t keep, double scale) {
   DNET_CHECK(w.dim() == 2 && is_f32(w) && w.is_contiguous(), "w fp32 [R, W]");
   const int R = w.size(0), W = w.size(1);
   const int64_t T = we.size(0), E = we.size(1);
@@ -457,7 +510,13 @@ void moe_router(c10::optional<torch::Tensor> x, torch::Tensor w,
   if (gate.has_value())
     DNET_CHECK(is_f32(*gate) && gate->is_contiguous() && gate->numel() == T,
                "gate fp32 [T]");
-  const size_t lds = (size_t)R * sizeof(float);
+  DNET_CHECK(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups &&
+                 top <= keep * (E / groups), "expert groups");
+  if (corr.has_value())
+    DNET_CHECK(is_f32(*corr) && corr->is_contiguous() && corr->numel() == E,
+               "correction fp32 [E]");
+  const float* cp = corr.has_value() ? corr->data_ptr<float>() : nullptr;
+  const size_t lds = (size_t)(R + E + groups) * sizeof(float);
   DNET_CHECK(lds <= 60 * 1024, "moe_router: too many experts");
   if (T == 0) return;
   float* gp = gate.has_value() ? gate->data_ptr<float>() : nullptr;
@@ -466,7 +525,8 @@ void moe_router(c10::optional<torch::Tensor> x, torch::Tensor w,
   hipLaunchKernelGGL((moe_router_kernel<TT>), dim3((unsigned)T), dim3(NT),    \
                      lds, st, XP, w.data_ptr<float>(), LP,                    \
                      idx.data_ptr<int>(), val.data_ptr<float>(),              \
-                     we.data_ptr<float>(), gp, W, (int)E, R, top)
+                     we.data_ptr<float>(), gp, cp, W, (int)E, R, top,         \
+                     (int)groups, (int)keep, (float)scale)
   if (x.has_value()) {
     DNET_CHECK(x->dim() == 2 && x->is_contiguous() && x->size(0) == T &&
                    x->size(1) == W, "x [T, W]");
@@ -526,25 +586,43 @@ void moe_gather(torch::Tensor x, torch::Tensor order, torch::Tensor val,
                        scale.data_ptr<float>(), top, bytes);
 }
 
+// Routed rows of `x` [T, K] through the gated experts w [E, 2N, K]: shapes
+static void check_gated(const torch::Tensor& x, const torch::Tensor& w,
+                        const torch::Tensor& we, const torch::Tensor& act) {
+  const int64_t T = x.size(0), K = x.size(1), E = w.size(0), N = w.size(1) / 2;
+  DNET_CHECK(is_bf16(x) && is_bf16(w) && is_bf16(act) && is_f32(we) &&
+                 x.is_contiguous() && w.is_contiguous() &&
+                 act.is_contiguous() && we.is_contiguous(),
+             "gated expert rows: contiguous bf16, we fp32");
+  DNET_CHECK(x.dim() == 2 && w.dim() == 3 && w.size(1) % 2 == 0 &&
+                 w.size(2) == K && we.dim() == 2 && we.size(0) == T &&
+                 we.size(1) == E && act.dim() == 3 && act.size(0) == E &&
+                 act.size(1) == T && act.size(2) == N && K % 8 == 0 && K > 0 &&
+                 N > 0, "gated expert rows: shapes");
+}
+
 static void rows_launch(const torch::Tensor& x, const torch::Tensor& w,
                         const torch::Tensor& we, torch::Tensor& out, int64_t T,
-                        int64_t K, int64_t N, int kind, int64_t x_expert) {
+                        int64_t K, int64_t N, int kind, int64_t x_expert,
+                        float alpha = 0.f, float limit = 0.f) {
   const int64_t E = we.size(1);
   auto st = current_stream();
 #define RL(MM, NF, NW, UU, GG)                                                \
   hipLaunchKernelGGL((moe_rows_kernel<MM, NF, NW, UU, GG>),                   \
-                     dim3((unsigned)cdiv(N, GG == kGlu ? NF * 8 : NF * 16),           \
+                     dim3((unsigned)cdiv(N, GG == kGlu || GG == kClampGlu     \
+                                                ? NF * 8 : NF * 16),          \
                           (unsigned)cdiv(T, 16 * MM), (unsigned)E),           \
                      dim3(NW * 64), 0, st, (const short*)x.data_ptr(),        \
                      (const short*)w.data_ptr(), we.data_ptr<float>(),        \
                      (short*)out.data_ptr(), (int)K, (int)N, (int)E, (int)T,  \
-                     x_expert)
+                     x_expert, alpha, limit)
   // shapes measured at experts of 4096 x 3072 to 5120 x 12800: few rows want
   // more workgroups (narrow column tiles)
 #define RL_K(MM, NF, NW, UU)                            \
   do {                                                  \
     if (kind == kGlu) RL(MM, NF, NW, UU, kGlu);         \
     else if (kind == kReluSq) RL(MM, NF, NW, UU, kReluSq); \
+    else if (kind == kClampGlu) RL(MM, NF, NW, UU, kClampGlu); \
     else RL(MM, NF, NW, UU, kPlain);                    \
   } while (0)
   if (T <= 2 && kind == kPlain) RL(1, 1, 8, 4, kPlain);
@@ -557,18 +635,17 @@ static void rows_launch(const torch::Tensor& x, const torch::Tensor& w,
 
 void moe_gateup_rows(torch::Tensor x, torch::Tensor w, torch::Tensor we,
                      torch::Tensor act) {
-  const int64_t T = x.size(0), K = x.size(1), E = w.size(0), N = w.size(1) / 2;
-  DNET_CHECK(is_bf16(x) && is_bf16(w) && is_bf16(act) && is_f32(we) &&
-                 x.is_contiguous() && w.is_contiguous() &&
-                 act.is_contiguous() && we.is_contiguous(),
-             "moe_gateup_rows: contiguous bf16, we fp32");
-  DNET_CHECK(x.dim() == 2 && w.dim() == 3 && w.size(1) % 2 == 0 &&
-                 w.size(2) == K && we.dim() == 2 && we.size(0) == T &&
-                 we.size(1) == E && act.dim() == 3 && act.size(0) == E &&
-                 act.size(1) == T && act.size(2) == N && K % 8 == 0 && K > 0 &&
-                 N > 0, "moe_gateup_rows: shapes");
-  if (T == 0) return;
-  rows_launch(x, w, we, act, T, K, N, kGlu, 0);
+  check_gated(x, w, we, act);
+  if (x.size(0) == 0) return;
+  rows_launch(x, w, we, act, x.size(0), x.size(1), w.size(1) / 2, kGlu, 0);
+}
+
+void moe_clamped_rows(torch::Tensor x, torch::Tensor w, torch::Tensor we,
+                      torch::Tensor act, double alpha, double limit) {
+  check_gated(x, w, we, act);
+  if (x.size(0) == 0) return;
+  rows_launch(x, w, we, act, x.size(0), x.size(1), w.size(1) / 2, kClampGlu, 0,
+              (float)alpha, (float)limit);
 }
 
 void moe_up_rows(torch::Tensor x, torch::Tensor w, torch::Tensor we,

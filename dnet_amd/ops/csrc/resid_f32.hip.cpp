@@ -12,7 +12,7 @@
 //   resid_branches_rmsnorm  h += coef*(nrm(a) + nrm(b)) + f with optional
 //                     RMS-normalized branches, next norm and a cast copy of h
 //   gated_group_rmsnorm     grouped RMSNorm with a silu / sigmoid gate
-//   act_slice, gelu_gather_mul, clamped_glu   small element-wise steps
+//   act_slice, gelu_gather_mul   small element-wise steps
 //
 // One workgroup per token row; statistics are block-reduced in fp32. "short"
 // stands for bf16 bits throughout.
@@ -415,8 +415,8 @@ template <typename TG, typename TO>
 __global__ __launch_bounds__(256) void gated_group_rmsnorm_kernel(
     const float* __restrict__ y, const TG* __restrict__ gate_src,
     const int64_t gld, const int gcol0, const float* __restrict__ w,
-    TO* __restrict__ out, const int N, const int groups, const float eps,
-    const bool gate_silu, const bool gate_first) {
+    TO* __restrict__ out, const int64_t old, const int N, const int groups,
+    const float eps, const bool gate_silu, const bool gate_first) {
   const int wid = threadIdx.x / kWave, lane = threadIdx.x & (kWave - 1);
   const int64_t row = blockIdx.y;
   const int grp = blockIdx.x * (blockDim.x / kWave) + wid;
@@ -436,7 +436,7 @@ __global__ __launch_bounds__(256) void gated_group_rmsnorm_kernel(
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
   const float r = 1.0f / sqrtf(ss / (float)gs + eps);
-  TO* orow = out + row * N + (int64_t)grp * gs;
+  TO* orow = out + row * old + (int64_t)grp * gs;
   const float* wr = w + (int64_t)grp * gs;
   for (int e = lane; e < gs; e += kWave) {
     const float g = ldf<TG>(gr + e);
@@ -455,8 +455,8 @@ template <typename TG, typename TO, int W>
 __global__ __launch_bounds__(256) void gated_group_rmsnorm_wide_kernel(
     const float* __restrict__ y, const TG* __restrict__ gate_src,
     const int64_t gld, const int gcol0, const float* __restrict__ w,
-    TO* __restrict__ out, const int N, const int groups, const float eps,
-    const bool gate_silu, const bool gate_first) {
+    TO* __restrict__ out, const int64_t old, const int N, const int groups,
+    const float eps, const bool gate_silu, const bool gate_first) {
   __shared__ float red[8];
   const int64_t row = blockIdx.y;
   const int grp = blockIdx.x;
@@ -477,7 +477,7 @@ __global__ __launch_bounds__(256) void gated_group_rmsnorm_wide_kernel(
   }
   ss = block_reduce_sum(ss, red);
   const float r = 1.0f / sqrtf(ss / (float)gs + eps);
-  TO* orow = out + row * N + (int64_t)grp * gs;
+  TO* orow = out + row * old + (int64_t)grp * gs;
   const float* wr = w + (int64_t)grp * gs;
   for (int e = threadIdx.x * W; e < gs; e += blockDim.x * W) {
     vecf<W> v = ldw<W, float>(yr + e);
@@ -536,21 +536,6 @@ __global__ __launch_bounds__(256) void gelu_gather_mul_kernel(
         0.5f * v *
         (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
     stf<T>(y + i, g * ldf<T>(table + tok * tld + col0 + c));
-  }
-}
-
-template <typename T>
-__global__ __launch_bounds__(256) void clamped_glu_kernel(
-    const T* __restrict__ gu, T* __restrict__ y, const int I,
-    const int64_t total, const float alpha, const float limit) {
-  for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total;
-       i += (int64_t)gridDim.x * blockDim.x) {
-    const int64_t row = i / I;
-    const int c = (int)(i % I);
-    const float g = fminf(ldf<T>(gu + row * 2 * I + c), limit);
-    const float u =
-        fminf(fmaxf(ldf<T>(gu + row * 2 * I + I + c), -limit), limit);
-    stf<T>(y + i, g * sigmoid_f(alpha * g) * (u + 1.0f));
   }
 }
 
@@ -781,20 +766,24 @@ void gated_group_rmsnorm(torch::Tensor y, torch::Tensor gate_src,
                  gate_src.size(0) == M && gate_col0 >= 0 &&
                  gate_col0 + N <= gate_src.size(1), "gate columns");
   DNET_CHECK(is_f32(w) && w.is_contiguous() && w.numel() == N, "w fp32 [N]");
-  DNET_CHECK(out.is_contiguous() && out.size(0) == M && out.size(1) == N,
+  // (the output rows may be a column range of a wider buffer)
+  DNET_CHECK(out.dim() == 2 && out.size(0) == M && out.size(1) == N &&
+                 out.stride(1) == 1 && (M <= 1 || out.stride(0) >= N),
              "out [M, N]");
   if (M == 0) return;
   auto st = current_stream();
   const int gs = N / (int)groups;
   const bool wide = gs >= 1024;
-  const bool v4 = gs % 4 == 0 && gate_src.size(1) % 4 == 0 && gate_col0 % 4 == 0;
+  const bool v4 = gs % 4 == 0 && gate_src.size(1) % 4 == 0 &&
+                  gate_col0 % 4 == 0 && out.stride(0) % 4 == 0 &&
+                  out.storage_offset() % 4 == 0;
   const dim3 grid(wide ? (unsigned)groups : (unsigned)((groups + 3) / 4),
                   (unsigned)M);
 #define GG_ARGS(TG, TO)                                                      \
   grid, dim3(256), 0, st, y.data_ptr<float>(),                               \
       (const TG*)gate_src.data_ptr(), gate_src.size(1), (int)gate_col0,      \
-      w.data_ptr<float>(), (TO*)out.data_ptr(), N, (int)groups, (float)eps,  \
-      gate_silu, gate_first
+      w.data_ptr<float>(), (TO*)out.data_ptr(), out.stride(0), N,            \
+      (int)groups, (float)eps, gate_silu, gate_first
 #define GG(TG, TO)                                                           \
   do {                                                                       \
     if (wide && v4)                                                          \
@@ -870,28 +859,6 @@ void gelu_gather_mul(torch::Tensor z, torch::Tensor table,
                        table.size(0), tokens.data_ptr<int64_t>(), (int)col0,
                        (float*)y.data_ptr(), (int)z.size(1), total);
   else DNET_CHECK(false, "gelu_gather_mul: dtype");
-}
-
-void clamped_glu(torch::Tensor gu, torch::Tensor y, double alpha,
-                 double limit) {
-  DNET_CHECK(gu.dim() == 2 && gu.is_contiguous() && gu.size(1) % 2 == 0 &&
-                 y.is_contiguous() && y.size(0) == gu.size(0) &&
-                 y.size(1) * 2 == gu.size(1) &&
-                 y.scalar_type() == gu.scalar_type(), "clamped_glu: shapes");
-  const int64_t total = y.numel();
-  if (total == 0) return;
-  auto st = current_stream();
-  if (is_bf16(gu))
-    hipLaunchKernelGGL((clamped_glu_kernel<short>), dim3(ew_blocks(total)),
-                       dim3(256), 0, st, (const short*)gu.data_ptr(),
-                       (short*)y.data_ptr(), (int)y.size(1), total,
-                       (float)alpha, (float)limit);
-  else if (is_f32(gu))
-    hipLaunchKernelGGL((clamped_glu_kernel<float>), dim3(ew_blocks(total)),
-                       dim3(256), 0, st, (const float*)gu.data_ptr(),
-                       (float*)y.data_ptr(), (int)y.size(1), total,
-                       (float)alpha, (float)limit);
-  else DNET_CHECK(false, "clamped_glu: dtype");
 }
 
 }  // namespace dnet

@@ -387,18 +387,24 @@ __global__ __launch_bounds__(256) void cache_append_kernel(
 }
 
 // ---- gated activations ---------------------------------------------------------
-template <bool FAST, bool GELU> __device__ __forceinline__ float act_x(float g) {
-  if constexpr (GELU) {
+constexpr int kActSilu = 0, kActGelu = 1, kActClamp = 2;
+
+template <bool FAST, int KIND> __device__ __forceinline__ float act_x(float g) {
+  if constexpr (KIND == kActGelu) {
     const float k = 0.7978845608028654f;           // sqrt(2 / pi)
     return 0.5f * g * (1.f + tanh_x<FAST>(k * (g + 0.044715f * g * g * g)));
   }
   return g * sigmoid_x<FAST>(g);
 }
 
-template <typename T, int V, bool GELU>
+// silu, tanh-gelu: act(s g) * (s u), the row factor s on the inputs. Clamped:
+// g' sigmoid(alpha g') (u' + 1) s with g' = min(g, limit), u' = u clamped to
+// +-limit, the factor on the result.
+template <typename T, int V, int KIND>
 __global__ __launch_bounds__(256) void gated_act_kernel(
     const T* __restrict__ gu, const float* __restrict__ scale,
-    T* __restrict__ y, const int I, const int64_t total) {
+    T* __restrict__ y, const int I, const int64_t total, const float alpha,
+    const float limit) {
   constexpr bool FAST = sizeof(T) == 2;
   for (int64_t idx = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x) * V;
        idx < total; idx += (int64_t)gridDim.x * blockDim.x * V) {
@@ -408,8 +414,15 @@ __global__ __launch_bounds__(256) void gated_act_kernel(
     const vec<V> gv = ldv<V, T>(gu + row * 2 * I + c);
     vec<V> uv = ldv<V, T>(gu + row * 2 * I + I + c);
 #pragma unroll
-    for (int j = 0; j < V; ++j)
-      uv.v[j] = act_x<FAST, GELU>(gv.v[j] * s) * (uv.v[j] * s);
+    for (int j = 0; j < V; ++j) {
+      if constexpr (KIND == kActClamp) {
+        const float g = fminf(gv.v[j], limit);
+        const float u = fminf(fmaxf(uv.v[j], -limit), limit);
+        uv.v[j] = g * sigmoid_x<FAST>(alpha * g) * (u + 1.f) * s;
+      } else {
+        uv.v[j] = act_x<FAST, KIND>(gv.v[j] * s) * (uv.v[j] * s);
+      }
+    }
     stv<V, T>(y + idx, uv);
   }
 }
@@ -552,12 +565,12 @@ void cache_append(torch::Tensor src, int64_t col0, torch::Tensor cache,
 }
 
 void gated_act(torch::Tensor gu, c10::optional<torch::Tensor> scale,
-               torch::Tensor y, int64_t kind) {
+               torch::Tensor y, int64_t kind, double alpha, double limit) {
   DNET_CHECK(gu.dim() == 2 && gu.is_contiguous() && y.dim() == 2 &&
                  y.is_contiguous() && y.size(0) == gu.size(0) &&
                  gu.size(1) == 2 * y.size(1) &&
                  y.scalar_type() == gu.scalar_type(), "gu [M, 2I], y [M, I]");
-  DNET_CHECK(kind == 0 || kind == 1, "gated_act: kind");
+  DNET_CHECK(kind >= 0 && kind <= 2, "gated_act: kind");
   const float* sp = nullptr;
   if (scale.has_value()) {
     DNET_CHECK(is_f32(*scale) && scale->is_contiguous() &&
@@ -573,8 +586,13 @@ void gated_act(torch::Tensor gu, c10::optional<torch::Tensor> scale,
                      dim3((unsigned)std::min<int64_t>(                        \
                          (total / VV + 255) / 256, 8192)),                    \
                      dim3(256), 0, st, (const TT*)gu.data_ptr(), sp,          \
-                     (TT*)y.data_ptr(), I, total)
-#define GA_K(TT, VV) do { if (kind == 1) GA(TT, VV, true); else GA(TT, VV, false); } while (0)
+                     (TT*)y.data_ptr(), I, total, (float)alpha, (float)limit)
+#define GA_K(TT, VV)                                 \
+  do {                                               \
+    if (kind == kActGelu) GA(TT, VV, kActGelu);      \
+    else if (kind == kActClamp) GA(TT, VV, kActClamp); \
+    else GA(TT, VV, kActSilu);                       \
+  } while (0)
   if (is_bf16(gu)) { if (I % 8 == 0) GA_K(short, 8); else GA_K(short, 1); }
   else if (is_f32(gu)) { if (I % 4 == 0) GA_K(float, 4); else GA_K(float, 1); }
   else DNET_CHECK(false, "gated_act: dtype");

@@ -587,7 +587,8 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
              temp=None, softcap: float = 0.0, dist_r1=None, dist_r2=None,
              sinks=None, window: int = 0, pool_k=None, pool_v=None,
              pool: int = 0, v_dim: int = 0, chunk: int = 0,
-             sig_bias=None) -> torch.Tensor:
+             sig_bias=None, keep: int = 0, gate=None, gate_col: int = 0,
+             gate_scale: float = 1.0, out=None) -> torch.Tensor:
     """Causal attention against the cache with score modifiers, all in
     fp32: s = q.k * scale * temp[h]; s = cap*tanh(s/cap);
     s -= r1[h] * ln(1 + r2[h] * (i-j)); softmax whose denominator also
@@ -606,7 +607,13 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
     ``chunk`` > 0: query i sees key j only inside its own block of ``chunk``
     positions (j >= (i // chunk) * chunk; blocks count from position 0).
     ``sig_bias`` fp32 [Hq]: no softmax; the weight of a visible key is
-    sigmoid(s + sig_bias[h]), not normalized over the keys."""
+    sigmoid(s + sig_bias[h]), not normalized over the keys.
+
+    ``keep`` > 0 (with a window): every query also sees the keys j < keep, at
+    their true positions and in the same softmax. ``gate`` [B*T, ld]: head h's
+    result is multiplied by gate_scale * sigmoid(gate[row, gate_col + h])
+    before it is rounded. ``out``: a column range of a wider buffer that takes
+    the result (padding rows are left alone)."""
     Hkv, D = kcache.shape[1], kcache.shape[3]
     if vcache is None:
         vcache = kcache[..., :v_dim]
@@ -615,8 +622,17 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
     B = M // T
     Hq = q.shape[1] // D
     G = Hq // Hkv
-    out = torch.zeros(M, Hq * Dv, dtype=q.dtype, device=q.device)
+    if out is None:
+        out = torch.zeros(M, Hq * Dv, dtype=q.dtype, device=q.device)
     p, ln, sl = _row_index(B, T, pos, lens, slots, q.device)
+
+    def put(b, n, o):                       # o [n, Hkv, G, Dv]
+        o = o.reshape(n, Hq, Dv)
+        if gate is not None:
+            g = gate[b * T:b * T + n, gate_col:gate_col + Hq].float()
+            o = o * (gate_scale * torch.sigmoid(g)).unsqueeze(-1)
+        out[b * T:b * T + n] = o.reshape(n, Hq * Dv).to(q.dtype)
+
     for b in range(B):
         n = int(min(ln[b], T))
         if n <= 0:
@@ -640,7 +656,7 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
                 * dist.clamp(min=0).float())
         dead = dist < 0
         if window and window > 0:
-            dead = dead | (dist >= window)
+            dead = dead | ((dist >= window) & (j >= keep))
         if chunk and chunk > 0:
             dead = dead | (j < torch.div(i, chunk, rounding_mode="floor")
                            * chunk)
@@ -648,8 +664,7 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
             assert not pool and sinks is None
             pr = torch.sigmoid(sc + sig_bias.float().view(Hkv, G, 1, 1))
             pr = pr.masked_fill(dead, 0.0)
-            o = torch.einsum("hgts,hsd->thgd", pr, vv)
-            out[b * T:b * T + n] = o.reshape(n, Hq * Dv).to(q.dtype)
+            put(b, n, torch.einsum("hgts,hsd->thgd", pr, vv))
             continue
         sc = sc.masked_fill(dead, float("-inf"))
         nb = 0
@@ -673,8 +688,7 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
             pr = torch.softmax(torch.cat([sc, sk], dim=-1), dim=-1)[..., :-1]
         else:
             pr = torch.softmax(sc, dim=-1)
-        o = torch.einsum("hgts,hsd->thgd", pr, vv)
-        out[b * T:b * T + n] = o.reshape(n, Hq * Dv).to(q.dtype)
+        put(b, n, torch.einsum("hgts,hsd->thgd", pr, vv))
     return out
 
 
@@ -1307,11 +1321,20 @@ def cache_append(src: torch.Tensor, col0: int, cache: torch.Tensor,
             .reshape(n, H, D).transpose(0, 1).to(cache.dtype)
 
 
-def gated_act(gu: torch.Tensor, act: str, scale=None) -> torch.Tensor:
+def gated_act(gu: torch.Tensor, act: str, scale=None, alpha: float = 1.0,
+              limit: float = 0.0) -> torch.Tensor:
     """gu [M, 2I] = [gate | up] -> act(gate) * up [M, I], fp32 math.
-    ``scale`` fp32 [M]: factor of the row's input, act(s gate) * (s up)."""
+    ``scale`` fp32 [M]: factor of the row's input, act(s gate) * (s up).
+    act "clamped": g sigmoid(alpha g) (u + 1) with g = min(gate, limit) and u =
+    up clamped to +-limit; ``scale`` is then a factor of the result."""
     i = gu.shape[-1] // 2
     f = gu.float()
+    if act == "clamped":
+        g = f[:, :i].clamp(max=limit)
+        y = g * torch.sigmoid(alpha * g) * (f[:, i:].clamp(-limit, limit) + 1)
+        if scale is not None:
+            y = y * scale.view(-1, 1)
+        return y.to(gu.dtype)
     if scale is not None:
         f = f * scale.view(-1, 1)
     g, u = f[:, :i], f[:, i:]
@@ -1320,16 +1343,36 @@ def gated_act(gu: torch.Tensor, act: str, scale=None) -> torch.Tensor:
     return (g * u).to(gu.dtype)
 
 
-def moe_router(x: torch.Tensor, w: torch.Tensor, E: int, top: int):
+def moe_router(x: torch.Tensor, w: torch.Tensor, E: int, top: int,
+               correction=None, groups: int = 1, keep: int = 1,
+               scale: float = 1.0):
     """Sigmoid router in fp32. x [T, W], w fp32 [E or E+1, W] (the last row,
     when there, is the shared expert's gate). Returns (idx int32 [T, top],
     val fp32 [T, top], we fp32 [T, E] with the values of the chosen experts
-    and 0 elsewhere, gate fp32 [T] or None). The choice is made on the logits
-    (the sigmoid keeps their order, and rounds large ones to equal)."""
+    and 0 elsewhere, gate fp32 [T] or None); a value is the expert's score
+    times ``scale``.
+
+    Plain routers choose by the logits (the sigmoid keeps their order, and
+    rounds large ones to equal). With ``correction`` fp32 [E] the choice is
+    made on score + correction; with ``groups`` > 1 only experts of the
+    ``keep`` best groups of neighbours can be chosen, a group's score being the
+    sum of its two largest choice scores."""
+    T = x.shape[0]
     z = x.float() @ w.t()
-    val, idx = torch.topk(z[:, :E], top, dim=-1)
-    val = torch.sigmoid(val)
-    we = torch.zeros_like(z[:, :E]).scatter_(1, idx, val)
+    s = torch.sigmoid(z[:, :E])
+    c = z[:, :E]
+    if correction is not None or groups > 1:
+        c = s if correction is None else s + correction
+    if groups > 1:
+        gc = c.view(T, groups, E // groups)
+        best = gc.topk(min(2, E // groups), dim=-1).values.sum(-1) \
+            .topk(keep, dim=-1).indices
+        on = torch.zeros(T, groups, dtype=torch.bool, device=x.device) \
+            .scatter_(1, best, True)
+        c = gc.masked_fill(~on.unsqueeze(-1), float("-inf")).reshape(T, E)
+    idx = torch.topk(c, top, dim=-1).indices
+    val = torch.gather(s, 1, idx) * scale
+    we = torch.zeros_like(s).scatter_(1, idx, val)
     gate = torch.sigmoid(z[:, E]) if w.shape[0] > E else None
     return idx.to(torch.int32), val, we, gate
 
@@ -1388,3 +1431,179 @@ def moe_down_rows(act: torch.Tensor, w: torch.Tensor,
     """Experts' second half: act [E, T, I], w [E, N, I] -> [E, T, N] in
     act's dtype (rows of experts nobody chose may hold anything)."""
     return torch.einsum("eti,eni->etn", act.float(), w.float()).to(act.dtype)
+
+
+def moe_clamped_rows(x: torch.Tensor, w: torch.Tensor, we: torch.Tensor,
+                     alpha: float, limit: float) -> torch.Tensor:
+    """Experts' first half on every row with a clamped gate, the routing
+    weight on the result: x [T, K], w [E, 2I, K], we [T, E] -> act [E, T, I]
+    in x's dtype (0 for rows that did not choose the expert)."""
+    z = torch.einsum("tk,eik->eti", x.float(), w.float())
+    i = z.shape[-1] // 2
+    g = z[..., :i].clamp(max=limit)
+    y = g * torch.sigmoid(alpha * g) * (z[..., i:].clamp(-limit, limit) + 1)
+    return (y * we.t().unsqueeze(-1)).to(x.dtype)
+
+
+# ---- biased / convolved attention projections, gated linear attention, matrix
+# memory (fedinex) ----
+
+def qkv_rope_append(src: torch.Tensor, col0: int, nq: int, nkv: int, d: int,
+                    dv: int, kcache: torch.Tensor, vcache: torch.Tensor,
+                    pos: torch.Tensor, T: int, lens=None, slots=None,
+                    bias=None, conv_w=None, conv_state=None, rot_freq=None,
+                    half: bool = False, vf=None, lam=None) -> torch.Tensor:
+    """Columns col0.. of src [B*T, ld] = [q (nq*d) | k (nkv*d) | v (nkv*dv)],
+    in this order: + ``bias`` fp32; causal convolution over time per channel
+    (``conv_w`` fp32 [C, taps], last tap on the token itself, no activation;
+    ``conv_state`` [Bc, taps-1, C] holds a slot's last inputs, zero before
+    position 0); rotation of q and k by position * rot_freq[i], pair i being
+    channels (2i, 2i+1) or, ``half``, (i, i + n); v <- (1 - lam) v + lam vf
+    (``lam`` fp32 [1]; ``vf``: this step's rows [B*T, nkv*dv] or another
+    layer's value cache, read at the token's own place). Keys and values go to
+    the cache, the queries are returned (rows of padding hold anything)."""
+    M = src.shape[0]
+    B = M // T
+    NQ, NK = nq * d, nkv * d
+    C = NQ + NK + nkv * dv
+    x = src[:, col0:col0 + C].float()
+    if bias is not None:
+        x = x + bias
+    p, ln, sl = _row_index(B, T, pos, lens, slots, src.device)
+    if conv_w is not None:
+        taps = conv_w.shape[1]
+        y = torch.zeros_like(x)
+        for b in range(B):
+            n = int(min(ln[b], T))
+            if n <= 0:
+                continue
+            p0, s = int(p[b]), int(sl[b])
+            tail = conv_state[s].float()
+            if p0 < taps - 1:               # inputs before position 0
+                tail = tail.clone()
+                tail[:taps - 1 - p0] = 0
+            u = torch.cat([tail, x[b * T:b * T + n]])
+            for j in range(taps):
+                y[b * T:b * T + n] += conv_w[:, j] * u[j:j + n]
+            conv_state[s] = u[n:].to(conv_state.dtype)
+        x = y
+    q = x[:, :NQ].view(M, nq, d)
+    k = x[:, NQ:NQ + NK].view(M, nkv, d)
+    v = x[:, NQ + NK:].view(M, nkv, dv)
+    if rot_freq is not None and rot_freq.numel():
+        n = rot_freq.numel()
+        at = (p.view(B, 1) + torch.arange(T, device=src.device)
+              ).reshape(M, 1).float()
+        ang = at * rot_freq.view(1, -1)
+        if half:
+            c, s_ = torch.cos(ang).unsqueeze(1), torch.sin(ang).unsqueeze(1)
+
+            def turn(a):
+                u, w = a[..., :n], a[..., n:2 * n]
+                return torch.cat([u * c - w * s_, w * c + u * s_,
+                                  a[..., 2 * n:]], dim=-1)
+        else:
+            def turn(a):
+                return rotate_pairs(a, ang)
+        q, k = turn(q), turn(k)
+    for b in range(B):
+        n = int(min(ln[b], T))
+        if n <= 0:
+            continue
+        p0, s = int(p[b]), int(sl[b])
+        kb = k[b * T:b * T + n].transpose(0, 1)
+        vb = v[b * T:b * T + n].transpose(0, 1)
+        if vf is not None:
+            f = (vf[b * T:b * T + n].view(n, nkv, dv).transpose(0, 1)
+                 if vf.dim() == 2 else vf[s, :, p0:p0 + n]).float()
+            vb = (1 - lam) * vb + lam * f
+        kcache[s, :, p0:p0 + n] = kb.to(kcache.dtype)
+        vcache[s, :, p0:p0 + n] = vb.to(vcache.dtype)
+    return q.reshape(M, NQ).to(src.dtype)
+
+
+def gla_scan(src: torch.Tensor, q0: int, k0: int, v0: int, a0: int,
+             a2t: torch.Tensor, ab: torch.Tensor, inv_tau: float,
+             qscale: float, state: torch.Tensor, pos: torch.Tensor, T: int,
+             lens=None, slots=None) -> torch.Tensor:
+    """Gated linear attention, fp32. Columns of src [B*T, ld]: q0, k0 (H*d),
+    v0 (H*dv), a0 (rank); decays sigmoid(a . a2t + ab)^inv_tau per key channel
+    (a2t fp32 [rank, H*d]); S <- diag(decay) S + k v^T, o = S^T (qscale q).
+    ``state`` fp32 [Bc, H, d, dv], zero at position 0. Returns fp32 [B*T,
+    H*dv] (padding rows zero)."""
+    M = src.shape[0]
+    B = M // T
+    _, H, d, dv = state.shape
+    out = torch.zeros(M, H * dv, dtype=torch.float32, device=src.device)
+    p, ln, sl = _row_index(B, T, pos, lens, slots, src.device)
+    for b in range(B):
+        n = int(min(ln[b], T))
+        if n <= 0:
+            continue
+        p0, s = int(p[b]), int(sl[b])
+        f = src[b * T:b * T + n].float()
+        q = (f[:, q0:q0 + H * d] * qscale).view(n, H, d)
+        k = f[:, k0:k0 + H * d].view(n, H, d)
+        v = f[:, v0:v0 + H * dv].view(n, H, dv)
+        z = f[:, a0:a0 + a2t.shape[0]] @ a2t + ab
+        decay = torch.exp(torch.nn.functional.logsigmoid(z) * inv_tau) \
+            .view(n, H, d)
+        S = state[s].clone() if p0 > 0 else torch.zeros_like(state[s])
+        for t in range(n):
+            S = decay[t].unsqueeze(-1) * S \
+                + k[t].unsqueeze(-1) * v[t].unsqueeze(-2)
+            out[b * T + t] = torch.einsum("hdv,hd->hv", S, q[t]).reshape(-1)
+        state[s] = S
+    return out
+
+
+def mlstm_scan(src: torch.Tensor, q0: int, k0: int, v0: int, i0: int, f0: int,
+               ib: torch.Tensor, fb: torch.Tensor, cap: float, qscale: float,
+               state: torch.Tensor, nst: torch.Tensor, mst: torch.Tensor,
+               pos: torch.Tensor, T: int, lens=None,
+               slots=None) -> torch.Tensor:
+    """Matrix memory with exponential gates and a running maximum, fp32.
+    Columns of src [B*T, ld]: q0, k0 (H*d), v0 (H*dv), i0, f0 (H); log gates
+    i = cap tanh((. + ib) / cap), f = logsigmoid(cap tanh((. + fb) / cap));
+    m' = max(f + m, i); S <- exp(f + m - m') S + exp(i - m') k v^T, n like S
+    with k alone; o = S^T q / (max(|n . q|, exp(-m')) + 1e-6) with q times
+    ``qscale``. States fp32, zero at position 0: ``state`` [Bc, H, d, dv],
+    ``nst`` [Bc, H, tiles, d] and ``mst`` [Bc, H, tiles] (one copy per column
+    tile of the kernel). Returns fp32 [B*T, H*dv] (padding rows zero)."""
+    M = src.shape[0]
+    B = M // T
+    _, H, d, dv = state.shape
+    out = torch.zeros(M, H * dv, dtype=torch.float32, device=src.device)
+    p, ln, sl = _row_index(B, T, pos, lens, slots, src.device)
+    for b in range(B):
+        cnt = int(min(ln[b], T))
+        if cnt <= 0:
+            continue
+        p0, s = int(p[b]), int(sl[b])
+        x = src[b * T:b * T + cnt].float()
+        q = (x[:, q0:q0 + H * d] * qscale).view(cnt, H, d)
+        k = x[:, k0:k0 + H * d].view(cnt, H, d)
+        v = x[:, v0:v0 + H * dv].view(cnt, H, dv)
+        i = cap * torch.tanh((x[:, i0:i0 + H] + ib) / cap)
+        f = torch.nn.functional.logsigmoid(
+            cap * torch.tanh((x[:, f0:f0 + H] + fb) / cap))
+        if p0 > 0:
+            S, n, m = state[s].clone(), nst[s, :, 0].clone(), \
+                mst[s, :, 0].clone()
+        else:
+            S = torch.zeros_like(state[s])
+            n, m = torch.zeros_like(nst[s, :, 0]), \
+                torch.zeros_like(mst[s, :, 0])
+        for t in range(cnt):
+            mn = torch.maximum(f[t] + m, i[t])
+            keep, put = torch.exp(f[t] + m - mn), torch.exp(i[t] - mn)
+            S = keep.view(H, 1, 1) * S + put.view(H, 1, 1) \
+                * k[t].unsqueeze(-1) * v[t].unsqueeze(-2)
+            n = keep.view(H, 1) * n + put.view(H, 1) * k[t]
+            m = mn
+            den = torch.maximum((n * q[t]).sum(-1).abs(), torch.exp(-m)) \
+                + 1e-6
+            out[b * T + t] = (torch.einsum("hdv,hd->hv", S, q[t])
+                              / den.view(H, 1)).reshape(-1)
+        state[s], nst[s], mst[s] = S, n.unsqueeze(1), m.unsqueeze(1)
+    return out
