@@ -55,9 +55,26 @@ _COMPARE_SIZES = [("2k", 2048, 16, 4, 128, 8192),
 
 def _family_hf(fam, W, H, KV, D, FF, layers, vocab, args):
     """config.json-style description of ``fam`` at the given layer sizes."""
-    from dnet_amd.models.config import (gegorax_config, komizen_config,
-                                        lurisun_config, posudra_config,
-                                        turevik_config)
+    from dnet_amd.models.config import (fedinex_config, gegorax_config,
+                                        komizen_config, lurisun_config,
+                                        posudra_config, turevik_config)
+    if fam == "fedinex":
+        # windowed attention (half the prompt) with 4 kept first tokens and
+        # value mixing, convolved attention beside a matrix memory, gated
+        # linear attention in turn; recurrent heads of 64 x 128 state over the
+        # model width; dense clamped feed-forwards unless --compare-experts
+        # asks for a mixture in every second layer (experts in 4 groups, the
+        # best 2 eligible)
+        E = args.compare_experts
+        return fedinex_config(
+            W, vocab, "apg", layers=layers, heads=H, kv_heads=KV, dim=D,
+            vdim=D, rot_dims=D // 2, window=max(64, args.prompt_len // 2),
+            keep_first=4, left_heads=H, left_kv_heads=KV, left_dim=D,
+            left_vdim=D, conv=4, left_rot_dims=D // 2, mem_heads=W // 128,
+            mem_dim=64, mem_vdim=128, gla_heads=W // 128, gla_dim=64,
+            gla_vdim=128, ff=FF, limit=7.0, experts=E, top=min(4, E),
+            expert_ff=FF // 8, groups=4 if E >= 8 else 1,
+            keep_groups=2 if E >= 8 else 1)
     if fam == "turevik":
         # layers of four kinds in turn: latent attention with rows of its
         # own, two latent-attention layers on those rows, a minGRU over the
@@ -125,7 +142,7 @@ def _family_hf(fam, W, H, KV, D, FF, layers, vocab, args):
 # family -> the closest existing family it is measured beside
 _COMPARE_WITH = {"posudra": "qwen3", "gegorax": "posudra",
                  "komizen": "gegorax", "lurisun": "gegorax",
-                 "turevik": "komizen"}
+                 "turevik": "komizen", "fedinex": "gegorax"}
 
 
 def compare_family(args, device):
@@ -136,7 +153,9 @@ def compare_family(args, device):
     an fp32 residual with per-slot recurrent state; lurisun: gegorax —
     windowed attention beside linear recurrences with per-slot state, dense
     feed-forwards, fp32 residual; turevik: komizen — latent attention on
-    shared rows, recurrent layers with per-slot state, mixtures of experts)
+    shared rows, recurrent layers with per-slot state, mixtures of experts;
+    fedinex: gegorax — windowed attention, attention beside a recurrent mixer,
+    a linear recurrence, dense or clamped-expert feed-forwards, fp32 residual)
     at equal layer sizes, bf16, random weights. One JSON line; the default
     workload is untouched."""
     new, old = args.compare_family, _COMPARE_WITH[args.compare_family]
@@ -226,14 +245,14 @@ def main():
                          "enables host-DRAM weight streaming)")
     ap.add_argument("--compare-family", default="",
                     choices=["", "posudra", "gegorax", "komizen", "lurisun",
-                             "turevik"],
+                             "turevik", "fedinex"],
                     help="instead of the default workload: throughput of "
                          "this family beside its closest existing one at "
                          "equal layer sizes")
     ap.add_argument("--compare-layers", type=int, default=8)
     ap.add_argument("--compare-experts", type=int, default=0,
-                    help="gegorax: experts of the mixture feed-forward in "
-                         "every second layer (0 = dense feed-forwards); "
+                    help="gegorax, fedinex: experts of the mixture "
+                         "feed-forward in every second layer (0 = dense feed-forwards); "
                          "komizen, turevik: experts of every mixture (0 = 8)")
     ap.add_argument("--compare-prefill-batch", type=int, default=8)
     ap.add_argument("--compare-sizes", default="",

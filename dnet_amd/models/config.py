@@ -5,6 +5,7 @@ gpt-oss, deepseek-v2 — reference: src/dnet/core/models/*) with one dataclass.
 """
 from __future__ import annotations
 
+import copy
 from dataclasses import dataclass, field
 from typing import Optional
 
@@ -829,10 +830,11 @@ def fedinex_config(width: int, vocab: int, pattern: str = "apg",
     out = []
     for i in range(layers or len(pattern)):
         kind, m = mix[pattern[i % len(pattern)]]
-        out.append({"type": kind, "mixer": dict(m),
+        out.append({"type": kind, "mixer": m,
                     "mlp": moe if experts and i % 2 else dense})
+    # (layers share no dicts, so that a caller may edit one of them)
     return {"architecture": "Fedinex", "vocab": vocab, "width": width,
-            "norm": {"eps": eps}, "layers": out}
+            "norm": {"eps": eps}, "layers": [copy.deepcopy(s) for s in out]}
 
 
 # Known configs for synthetic benchmarking (random-init weights; no network).

@@ -413,13 +413,11 @@ class FedinexRingModel(RingModel):
         ops.attn_mod(q, kv.k[li], kv.v[li], pos, T, float(lf["scale"]), lens,
                      slots, gate=p, gate_col=c["lg"],
                      gate_scale=float(m["left_scale"]), out=y[:, :nl])
-        o = ops.mlstm_scan(p, c["rq"], c["rk"], c["rv"], c["ri"], c["rf"],
-                           lw.i_bias, lw.f_bias, float(rt["gate_cap"]),
-                           rt["dim"] ** -0.5, st["S"], st["n"], st["m"], pos,
-                           T, lens, slots)
-        ops.gated_group_rmsnorm(o, p, c["rg"], lw.mix_norm, rt["heads"],
-                                self.cfg.rms_eps, "sigmoid", False,
-                                self.wdtype, out=y[:, nl:])
+        ops.mlstm_heads(p, c["rq"], c["rk"], c["rv"], c["ri"], c["rf"],
+                        lw.i_bias, lw.f_bias, float(rt["gate_cap"]),
+                        rt["dim"] ** -0.5, st["S"], st["n"], st["m"], pos, T,
+                        lens, slots, lw.mix_norm, c["rg"], "sigmoid",
+                        self.cfg.rms_eps, out=y[:, nl:])
         return lw.o(y)
 
     def _gla(self, u, lw, lid, kv, pos, T, lens, slots, v_hop):
@@ -427,12 +425,10 @@ class FedinexRingModel(RingModel):
         H, d, dv = m["heads"], m["dim"], m["vdim"]
         p = lw.qkv(u)                              # [q | k | v | g | a1]
         g0 = 2 * H * d + H * dv
-        o = ops.gla_scan(p, 0, H * d, 2 * H * d, g0 + H * dv, lw.a2t, lw.a2_b,
-                         1.0 / float(m["tau"]), d ** -0.5,
-                         kv.state[kv.local[lid]]["S"], pos, T, lens, slots)
-        return lw.o(ops.gated_group_rmsnorm(
-            o, p, g0, lw.mix_norm, H, self.cfg.rms_eps, "silu", False,
-            self.wdtype))
+        return lw.o(ops.gla_heads(
+            p, 0, H * d, 2 * H * d, g0 + H * dv, lw.a2t, lw.a2_b,
+            1.0 / float(m["tau"]), d ** -0.5, kv.state[kv.local[lid]]["S"],
+            pos, T, lens, slots, lw.mix_norm, g0, "silu", self.cfg.rms_eps))
 
     def _moe(self, u, lw, ff, step: bool):
         """Routed experts, their results weighted. ``step``: a decode step,

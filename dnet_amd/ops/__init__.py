@@ -1133,3 +1133,45 @@ def mlstm_scan(src, q0: int, k0: int, v0: int, i0: int, f0: int, ib, fb,
         return o
     return ref.mlstm_scan(src, q0, k0, v0, i0, f0, ib, fb, cap, qscale, state,
                           nst, mst, pos, T, lens, slots)
+
+
+def _heads_out(src, state, out):
+    if out is not None:
+        return out
+    return torch.empty(src.shape[0], state.shape[1] * state.shape[3],
+                       dtype=src.dtype, device=src.device)
+
+
+def gla_heads(src, q0: int, k0: int, v0: int, a0: int, a2t, ab,
+              inv_tau: float, qscale: float, state, pos, T: int, lens, slots,
+              w, g0: int, gate_act: str, eps: float, out=None) -> torch.Tensor:
+    """``gla_scan`` with what follows it: per-head RMS norm, weight w [H*dv],
+    gate from columns g0.. of src, in src's dtype (``out``: a column range of
+    a wider buffer). One launch in decode steps."""
+    if src.is_cuda and T == 1:
+        out = _heads_out(src, state, out)
+        _native().gla_step(src, q0, k0, v0, a0, a2t, ab, inv_tau, qscale,
+                           state, w, g0, gate_act == "silu", eps, out, pos,
+                           lens, slots)
+        return out
+    o = gla_scan(src, q0, k0, v0, a0, a2t, ab, inv_tau, qscale, state, pos, T,
+                 lens, slots)
+    return gated_group_rmsnorm(o, src, g0, w, state.shape[1], eps, gate_act,
+                               False, src.dtype, out)
+
+
+def mlstm_heads(src, q0: int, k0: int, v0: int, i0: int, f0: int, ib, fb,
+                cap: float, qscale: float, state, nst, mst, pos, T: int, lens,
+                slots, w, g0: int, gate_act: str, eps: float,
+                out=None) -> torch.Tensor:
+    """``mlstm_scan`` with what follows it, as ``gla_heads``."""
+    if src.is_cuda and T == 1:
+        out = _heads_out(src, state, out)
+        _native().mlstm_step(src, q0, k0, v0, i0, f0, ib, fb, cap, qscale,
+                             state, nst, mst, w, g0, gate_act == "silu", eps,
+                             out, pos, lens, slots)
+        return out
+    o = mlstm_scan(src, q0, k0, v0, i0, f0, ib, fb, cap, qscale, state, nst,
+                   mst, pos, T, lens, slots)
+    return gated_group_rmsnorm(o, src, g0, w, state.shape[1], eps, gate_act,
+                               False, src.dtype, out)

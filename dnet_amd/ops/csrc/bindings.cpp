@@ -146,6 +146,19 @@ void gla_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0, int64_t a0,
               double qscale, torch::Tensor state, torch::Tensor o,
               torch::Tensor pos, c10::optional<torch::Tensor> lens,
               c10::optional<torch::Tensor> slots, int64_t T);
+void gla_step(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0, int64_t a0,
+              torch::Tensor a2t, torch::Tensor ab, double inv_tau,
+              double qscale, torch::Tensor state, torch::Tensor w, int64_t g0,
+              bool silu, double eps, torch::Tensor out, torch::Tensor pos,
+              c10::optional<torch::Tensor> lens,
+              c10::optional<torch::Tensor> slots);
+void mlstm_step(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0,
+                int64_t i0, int64_t f0, torch::Tensor ib, torch::Tensor fb,
+                double cap, double qscale, torch::Tensor state,
+                torch::Tensor nst, torch::Tensor mst, torch::Tensor w,
+                int64_t g0, bool silu, double eps, torch::Tensor out,
+                torch::Tensor pos, c10::optional<torch::Tensor> lens,
+                c10::optional<torch::Tensor> slots);
 void mlstm_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0,
                 int64_t i0, int64_t f0, torch::Tensor ib, torch::Tensor fb,
                 double cap, double qscale, torch::Tensor state,
@@ -362,6 +375,10 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "linear attention with a low-rank decay per key channel");
   m.def("mlstm_scan", &dnet::mlstm_scan,
         "matrix memory with exponential gates and a running maximum");
+  m.def("gla_step", &dnet::gla_step,
+        "decode step of gla_scan with head norm, weight and output gate");
+  m.def("mlstm_step", &dnet::mlstm_step,
+        "decode step of mlstm_scan with head norm, weight and output gate");
   m.def("moe_clamped_rows", &dnet::moe_clamped_rows,
         "clamped gated experts on a decode batch, routing weight on the "
         "result (matrix cores)");

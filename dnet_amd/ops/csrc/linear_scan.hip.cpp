@@ -23,6 +23,11 @@
 // (of ones) on a wave of its own, which also forms the gates and the running
 // maximum; every column tile keeps its own copy of n and m, so that no
 // workgroup reads what another one writes.
+//
+// Decode steps (one token per row) have a kernel of their own: a workgroup owns
+// a head of a batch row, streams its state once through 16 B accesses, and goes
+// on with what follows the recurrence: RMS norm of the head, weight, output
+// gate, one rounding into the next product's operand.
 #include "common.h"
 
 namespace dnet {
@@ -254,6 +259,179 @@ __global__ __launch_bounds__(1024) void linear_scan_kernel(const ScanArgs a) {
   if (ncol && lane == 0) *mp = m;
 }
 
+// ---- one decode step -----------------------------------------------------------
+// grid (H, B). Thread (row group, column lane): V neighbouring columns of every
+// RG-th state row, the first rows in flight while the gates are formed.
+struct StepTail {
+  const float* w;            // norm weight [H*dv]
+  void* out;                 // [B, H*dv], row stride out_ld
+  int64_t out_ld;
+  int g0, silu;              // gate columns of src
+  float eps;
+};
+
+template <typename T> __device__ __forceinline__ void stx(T* p, float v);
+template <> __device__ __forceinline__ void stx<float>(float* p, float v) { *p = v; }
+template <> __device__ __forceinline__ void stx<short>(short* p, float v) { *p = f2bits(v); }
+
+template <int V> struct vecf { float v[V]; };
+template <int V> __device__ __forceinline__ vecf<V> ldf(const float* p) {
+  vecf<V> r;
+  if constexpr (V == 4) {
+    const float4 t = *reinterpret_cast<const float4*>(p);
+    r.v[0] = t.x; r.v[1] = t.y; r.v[2] = t.z; r.v[3] = t.w;
+  } else {
+    r.v[0] = *p;
+  }
+  return r;
+}
+template <int V> __device__ __forceinline__ void stf(float* p, const vecf<V>& r) {
+  if constexpr (V == 4)
+    *reinterpret_cast<float4*>(p) = make_float4(r.v[0], r.v[1], r.v[2], r.v[3]);
+  else *p = r.v[0];
+}
+
+constexpr int kStepRows = 8;   // state rows of a thread in flight
+
+template <typename T, int V, int KIND>
+__global__ __launch_bounds__(256) void linear_step_kernel(const ScanArgs a,
+                                                          const StepTail e) {
+  const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
+  const int d = a.d, dv = a.dv;
+  T* op = reinterpret_cast<T*>(e.out) + b * e.out_ld + (int64_t)h * dv;
+  const int slot = a.slots ? a.slots[b] : b;
+  const int p0 = a.pos[b];
+  if ((a.lens && a.lens[b] <= 0) || slot < 0 || slot >= a.Bc || p0 < 0) {
+    for (int c = tid; c < dv; c += 256) stx<T>(op + c, 0.f);   // idle row
+    return;
+  }
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  float* sQ = sm;                           // [d]
+  float* sK = sQ + d;
+  float* sA = sK + d;                       // gla: decays
+  float* sP = sm + (3 * d + 3) / 4 * 4;     // [RG][columns of one pass]
+  __shared__ float red[8];
+  const T* src = reinterpret_cast<const T*>(a.src) + (int64_t)b * a.ld;
+  const int CT = (dv + V - 1) / V;          // column lanes of the head
+  const int CL = min(CT, 256);              // ... of one pass
+  const int RG = 256 / CL;
+  const int rg = tid / CL, cl = tid % CL;
+  float* sO = sP + RG * CL * V;             // [dv]
+  float* st = a.state + ((int64_t)slot * a.H + h) * d * dv;
+  const bool old = p0 > 0;
+
+  vecf<V> pre[kStepRows];
+#pragma unroll
+  for (int u = 0; u < kStepRows; ++u) {
+    const int row = rg + u * RG;
+#pragma unroll
+    for (int j = 0; j < V; ++j) pre[u].v[j] = 0.f;
+    if (old && rg < RG && row < d)
+      pre[u] = ldf<V>(st + (int64_t)row * dv + cl * V);
+  }
+  float keep = 1.f, put = 1.f, floor_ = 0.f, nq = 0.f;
+  if constexpr (KIND == kMlstm) {
+    float* mp = a.mst + ((int64_t)slot * a.H + h) * a.NT;
+    const float m = old ? *mp : 0.f;
+    const float i = a.cap * tanhf((ldx<T>(src + a.i0 + h) + a.ib[h]) / a.cap);
+    const float f = log_sigmoid(
+        a.cap * tanhf((ldx<T>(src + a.f0 + h) + a.fb[h]) / a.cap));
+    const float mn = fmaxf(f + m, i);
+    keep = expf(f + m - mn);
+    put = expf(i - mn);
+    floor_ = expf(-mn);
+    __syncthreads();                        // every thread has read m
+    if (tid < a.NT) mp[tid] = mn;
+    for (int t = tid + 256; t < a.NT; t += 256) mp[t] = mn;
+  }
+  for (int i = tid; i < d; i += 256) {
+    const float q = ldx<T>(src + a.q0 + h * d + i) * a.qscale;
+    const float k = ldx<T>(src + a.k0 + h * d + i);
+    sQ[i] = q;
+    sK[i] = k;
+    if constexpr (KIND == kGla) {
+      float z = a.ab[h * d + i];
+      const float* wp = a.a2t + h * d + i;
+#pragma unroll 16
+      for (int r = 0; r < a.rank; ++r)
+        z = fmaf(wp[(int64_t)r * a.H * d], ldx<T>(src + a.a0 + r), z);
+      sA[i] = expf(log_sigmoid(z) * a.inv_tau);
+    } else {
+      // the normalizer, every column tile's copy
+      float* np = a.nst + ((int64_t)slot * a.H + h) * a.NT * d + i;
+      const float nn = fmaf(put, k, keep * (old ? *np : 0.f));
+      for (int t = 0; t < a.NT; ++t) np[(int64_t)t * d] = nn;
+      nq = fmaf(nn, q, nq);
+    }
+  }
+  if constexpr (KIND == kMlstm) nq = block_reduce_sum(nq, red);
+  __syncthreads();
+  for (int c0 = 0; c0 < CT; c0 += CL) {     // one pass up to 256 V columns
+    const int col = (c0 + cl) * V;
+    const bool on = rg < RG && c0 + cl < CT;
+    vecf<V> v, acc;
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      v.v[j] = on ? ldx<T>(src + a.v0 + h * dv + col + j) * put : 0.f;
+      acc.v[j] = 0.f;
+    }
+    if (on)
+      for (int r0 = rg; r0 < d; r0 += RG * kStepRows) {
+        vecf<V> s[kStepRows];
+        const bool first = c0 == 0 && r0 == rg;
+#pragma unroll
+        for (int u = 0; u < kStepRows; ++u) {
+          const int row = r0 + u * RG;
+          s[u] = pre[u];
+          if (!first && row < d) {
+#pragma unroll
+            for (int j = 0; j < V; ++j) s[u].v[j] = 0.f;
+            if (old) s[u] = ldf<V>(st + (int64_t)row * dv + col);
+          }
+        }
+#pragma unroll
+        for (int u = 0; u < kStepRows; ++u) {
+          const int row = r0 + u * RG;
+          if (row >= d) continue;
+          const float k = sK[row], q = sQ[row];
+          const float g = KIND == kGla ? sA[row] : keep;
+#pragma unroll
+          for (int j = 0; j < V; ++j) {
+            s[u].v[j] = fmaf(k, v.v[j], g * s[u].v[j]);
+            acc.v[j] = fmaf(s[u].v[j], q, acc.v[j]);
+          }
+          stf<V>(st + (int64_t)row * dv + col, s[u]);
+        }
+      }
+    __syncthreads();                        // sP of the last pass consumed
+    if (on)
+#pragma unroll
+      for (int j = 0; j < V; ++j) sP[(rg * CL + cl) * V + j] = acc.v[j];
+    __syncthreads();
+    for (int c = tid; c < CL * V && c0 * V + c < dv; c += 256) {
+      float o = 0.f;
+      for (int r = 0; r < RG; ++r) o += sP[r * CL * V + c];
+      sO[c0 * V + c] = o;
+    }
+  }
+  __syncthreads();
+  float inv = 1.f;
+  if constexpr (KIND == kMlstm) inv = 1.f / (fmaxf(fabsf(nq), floor_) + kDenEps);
+  float ss = 0.f;
+  for (int c = tid; c < dv; c += 256) {
+    const float o = sO[c] * inv;
+    ss = fmaf(o, o, ss);
+  }
+  ss = block_reduce_sum(ss, red);
+  const float r = inv / sqrtf(ss / (float)dv + e.eps);
+  for (int c = tid; c < dv; c += 256) {
+    const float g = ldx<T>(src + e.g0 + h * dv + c);
+    float s = 1.f / (1.f + expf(-g));
+    if (e.silu) s *= g;
+    stx<T>(op + c, sO[c] * r * e.w[h * dv + c] * s);
+  }
+}
+
 const int* idx32(const torch::Tensor& t, int64_t n) {
   DNET_CHECK(t.scalar_type() == torch::kInt32 && t.is_contiguous() &&
                  t.numel() >= n, "int32 index tensor [B]");
@@ -265,13 +443,13 @@ const float* f32p(const torch::Tensor& t, int64_t n, const char* what) {
   return t.data_ptr<float>();
 }
 
-// shared part of the two entry points: checks, geometry, launch shape
-void scan_launch(ScanArgs& a, int kind, const torch::Tensor& src, int64_t q0,
-                 int64_t k0, int64_t v0, double qscale, torch::Tensor& state,
-                 torch::Tensor& o, const torch::Tensor& pos,
-                 const c10::optional<torch::Tensor>& lens,
-                 const c10::optional<torch::Tensor>& slots, int64_t T,
-                 int64_t NT) {
+// shared part of the entry points: checks and geometry
+void fill_args(ScanArgs& a, const torch::Tensor& src, int64_t q0, int64_t k0,
+               int64_t v0, double qscale, torch::Tensor& state,
+               const torch::Tensor& pos,
+               const c10::optional<torch::Tensor>& lens,
+               const c10::optional<torch::Tensor>& slots, int64_t T,
+               int64_t NT) {
   const int64_t M = src.size(0), ld = src.size(1);
   DNET_CHECK(src.dim() == 2 && src.is_contiguous() &&
                  (is_bf16(src) || is_f32(src)), "src [B*T, ld]");
@@ -282,20 +460,26 @@ void scan_launch(ScanArgs& a, int kind, const torch::Tensor& src, int64_t q0,
   const int64_t H = state.size(1), d = state.size(2), dv = state.size(3);
   DNET_CHECK(q0 >= 0 && k0 >= 0 && v0 >= 0 && q0 + H * d <= ld &&
                  k0 + H * d <= ld && v0 + H * dv <= ld, "src columns");
-  DNET_CHECK(is_f32(o) && o.is_contiguous() && o.size(0) == M &&
-                 o.size(1) == H * dv, "o fp32 [B*T, H*dv]");
   DNET_CHECK(d >= 1 && d <= 512 && dv >= 1, "1 <= head size <= 512");
   if (!slots.has_value()) DNET_CHECK(B <= state.size(0), "more rows than slots");
-  if (M == 0) return;
   a.src = src.data_ptr();
   a.state = state.data_ptr<float>();
-  a.o = o.data_ptr<float>();
   a.pos = idx32(pos, B);
   a.lens = lens.has_value() ? idx32(*lens, B) : nullptr;
   a.slots = slots.has_value() ? idx32(*slots, B) : nullptr;
   a.ld = ld; a.q0 = (int)q0; a.k0 = (int)k0; a.v0 = (int)v0;
   a.T = (int)T; a.Bc = (int)state.size(0); a.H = (int)H; a.d = (int)d;
   a.dv = (int)dv; a.qscale = (float)qscale; a.NT = (int)NT;
+}
+
+void scan_launch(ScanArgs& a, int kind, const torch::Tensor& src,
+                 torch::Tensor& o) {
+  const int64_t M = src.size(0), B = M / a.T, T = a.T, NT = a.NT;
+  const int64_t H = a.H, d = a.d, dv = a.dv;
+  DNET_CHECK(is_f32(o) && o.is_contiguous() && o.size(0) == M &&
+                 o.size(1) == H * dv, "o fp32 [B*T, H*dv]");
+  if (M == 0) return;
+  a.o = o.data_ptr<float>();
   const int R = d <= 32 ? 8 : (d <= 128 ? 16 : 32);
   a.NS = 1;
   while (a.NS * R < d) a.NS *= 2;           // power of two, <= 16
@@ -331,15 +515,53 @@ void scan_launch(ScanArgs& a, int kind, const torch::Tensor& src, int64_t q0,
 #undef LS
 }
 
-}  // namespace
+// decode step of either kind with the head's norm, weight and output gate
+void step_launch(ScanArgs& a, int kind, const torch::Tensor& src,
+                 const torch::Tensor& w, int64_t g0, bool silu, double eps,
+                 torch::Tensor& out) {
+  const int64_t B = src.size(0), n = (int64_t)a.H * a.dv;
+  StepTail e;
+  e.w = f32p(w, n, "norm weight fp32 [H*dv]");
+  DNET_CHECK(g0 >= 0 && g0 + n <= src.size(1), "gate columns");
+  DNET_CHECK(out.dim() == 2 && out.size(0) == B && out.size(1) == n &&
+                 out.stride(1) == 1 && (B <= 1 || out.stride(0) >= n) &&
+                 out.scalar_type() == src.scalar_type(), "out [B, H*dv]");
+  if (B == 0) return;
+  e.out = out.data_ptr();
+  e.out_ld = out.stride(0);
+  e.g0 = (int)g0;
+  e.silu = silu ? 1 : 0;
+  e.eps = (float)eps;
+  const bool v4 = a.dv % 4 == 0;
+  const int V = v4 ? 4 : 1;
+  const int CL = std::min((a.dv + V - 1) / V, 256);
+  const size_t lds =
+      ((3 * a.d + 3) / 4 * 4 + (256 / CL) * CL * V + a.dv) * sizeof(float);
+  DNET_CHECK(lds <= 60 * 1024, "linear_step: sizes exceed LDS");
+  const dim3 grid((unsigned)a.H, (unsigned)B);
+  auto st = current_stream();
+#define LP(TT, VV, KK)                                                        \
+  hipLaunchKernelGGL((linear_step_kernel<TT, VV, KK>), grid, dim3(256), lds,  \
+                     st, a, e)
+#define LP_K(TT, VV) do { if (kind == kGla) LP(TT, VV, kGla); else LP(TT, VV, kMlstm); } while (0)
+#define LP_V(TT) do { if (v4) LP_K(TT, 4); else LP_K(TT, 1); } while (0)
+  if (is_bf16(src)) LP_V(short); else LP_V(float);
+#undef LP_V
+#undef LP_K
+#undef LP
+}
 
-void gla_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0, int64_t a0,
-              torch::Tensor a2t, torch::Tensor ab, double inv_tau,
-              double qscale, torch::Tensor state, torch::Tensor o,
-              torch::Tensor pos, c10::optional<torch::Tensor> lens,
-              c10::optional<torch::Tensor> slots, int64_t T) {
+ScanArgs gla_args(const torch::Tensor& src, int64_t q0, int64_t k0, int64_t v0,
+                  int64_t a0, const torch::Tensor& a2t, const torch::Tensor& ab,
+                  double inv_tau, double qscale, torch::Tensor& state,
+                  const torch::Tensor& pos,
+                  const c10::optional<torch::Tensor>& lens,
+                  const c10::optional<torch::Tensor>& slots, int64_t T) {
   ScanArgs a = {};
-  const int64_t n = state.size(1) * state.size(2);
+  // column tiles of up to 64
+  fill_args(a, src, q0, k0, v0, qscale, state, pos, lens, slots, T,
+            (state.size(3) + 63) / 64);
+  const int64_t n = (int64_t)a.H * a.d;
   DNET_CHECK(a2t.dim() == 2 && a2t.size(1) == n, "a2t fp32 [rank, H*d]");
   a.rank = (int)a2t.size(0);
   DNET_CHECK(a.rank >= 1 && a.rank <= 2048 && a0 >= 0 &&
@@ -348,24 +570,24 @@ void gla_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0, int64_t a0,
   a.ab = f32p(ab, n, "ab fp32 [H*d]");
   a.a0 = (int)a0;
   a.inv_tau = (float)inv_tau;
-  // column tiles of up to 64
-  const int64_t NT = (state.size(3) + 63) / 64;
-  scan_launch(a, kGla, src, q0, k0, v0, qscale, state, o, pos, lens, slots, T,
-              NT);
+  return a;
 }
 
-void mlstm_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0,
-                int64_t i0, int64_t f0, torch::Tensor ib, torch::Tensor fb,
-                double cap, double qscale, torch::Tensor state,
-                torch::Tensor nst, torch::Tensor mst, torch::Tensor o,
-                torch::Tensor pos, c10::optional<torch::Tensor> lens,
-                c10::optional<torch::Tensor> slots, int64_t T) {
+ScanArgs mlstm_args(const torch::Tensor& src, int64_t q0, int64_t k0,
+                    int64_t v0, int64_t i0, int64_t f0, const torch::Tensor& ib,
+                    const torch::Tensor& fb, double cap, double qscale,
+                    torch::Tensor& state, torch::Tensor& nst,
+                    torch::Tensor& mst, const torch::Tensor& pos,
+                    const c10::optional<torch::Tensor>& lens,
+                    const c10::optional<torch::Tensor>& slots, int64_t T) {
   ScanArgs a = {};
-  const int64_t Bc = state.size(0), H = state.size(1), d = state.size(2);
-  DNET_CHECK(nst.dim() == 4 && nst.size(0) == Bc && nst.size(1) == H &&
-                 nst.size(3) == d, "n fp32 [Bc, H, tiles, d]");
+  DNET_CHECK(nst.dim() == 4, "n fp32 [Bc, H, tiles, d]");
   const int64_t NT = nst.size(2);
-  DNET_CHECK(NT >= 1 && (state.size(3) + NT - 1) / NT <= 64, "column tiles");
+  fill_args(a, src, q0, k0, v0, qscale, state, pos, lens, slots, T, NT);
+  const int64_t Bc = a.Bc, H = a.H, d = a.d;
+  DNET_CHECK(nst.size(0) == Bc && nst.size(1) == H && nst.size(3) == d &&
+                 NT >= 1 && (a.dv + NT - 1) / NT <= 64,
+             "n fp32 [Bc, H, tiles, d], tiles of up to 64 columns");
   f32p(nst, Bc * H * NT * d, "n fp32 [Bc, H, tiles, d]");
   f32p(mst, Bc * H * NT, "m fp32 [Bc, H, tiles]");
   a.nst = nst.data_ptr<float>();
@@ -376,8 +598,53 @@ void mlstm_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0,
                  f0 + H <= src.size(1), "gate columns");
   DNET_CHECK(cap > 0, "gate cap");
   a.i0 = (int)i0; a.f0 = (int)f0; a.cap = (float)cap;
-  scan_launch(a, kMlstm, src, q0, k0, v0, qscale, state, o,
-              pos, lens, slots, T, NT);
+  return a;
+}
+
+}  // namespace
+
+void gla_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0, int64_t a0,
+              torch::Tensor a2t, torch::Tensor ab, double inv_tau,
+              double qscale, torch::Tensor state, torch::Tensor o,
+              torch::Tensor pos, c10::optional<torch::Tensor> lens,
+              c10::optional<torch::Tensor> slots, int64_t T) {
+  ScanArgs a = gla_args(src, q0, k0, v0, a0, a2t, ab, inv_tau, qscale, state,
+                        pos, lens, slots, T);
+  scan_launch(a, kGla, src, o);
+}
+
+void gla_step(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0, int64_t a0,
+              torch::Tensor a2t, torch::Tensor ab, double inv_tau,
+              double qscale, torch::Tensor state, torch::Tensor w, int64_t g0,
+              bool silu, double eps, torch::Tensor out, torch::Tensor pos,
+              c10::optional<torch::Tensor> lens,
+              c10::optional<torch::Tensor> slots) {
+  ScanArgs a = gla_args(src, q0, k0, v0, a0, a2t, ab, inv_tau, qscale, state,
+                        pos, lens, slots, 1);
+  step_launch(a, kGla, src, w, g0, silu, eps, out);
+}
+
+void mlstm_scan(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0,
+                int64_t i0, int64_t f0, torch::Tensor ib, torch::Tensor fb,
+                double cap, double qscale, torch::Tensor state,
+                torch::Tensor nst, torch::Tensor mst, torch::Tensor o,
+                torch::Tensor pos, c10::optional<torch::Tensor> lens,
+                c10::optional<torch::Tensor> slots, int64_t T) {
+  ScanArgs a = mlstm_args(src, q0, k0, v0, i0, f0, ib, fb, cap, qscale, state,
+                          nst, mst, pos, lens, slots, T);
+  scan_launch(a, kMlstm, src, o);
+}
+
+void mlstm_step(torch::Tensor src, int64_t q0, int64_t k0, int64_t v0,
+                int64_t i0, int64_t f0, torch::Tensor ib, torch::Tensor fb,
+                double cap, double qscale, torch::Tensor state,
+                torch::Tensor nst, torch::Tensor mst, torch::Tensor w,
+                int64_t g0, bool silu, double eps, torch::Tensor out,
+                torch::Tensor pos, c10::optional<torch::Tensor> lens,
+                c10::optional<torch::Tensor> slots) {
+  ScanArgs a = mlstm_args(src, q0, k0, v0, i0, f0, ib, fb, cap, qscale, state,
+                          nst, mst, pos, lens, slots, 1);
+  step_launch(a, kMlstm, src, w, g0, silu, eps, out);
 }
 
 }  // namespace dnet

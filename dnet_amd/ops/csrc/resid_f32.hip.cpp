@@ -449,6 +449,46 @@ __global__ __launch_bounds__(256) void gated_group_rmsnorm_kernel(
   }
 }
 
+// Narrow groups (<= 256 channels, a multiple of 4): LPG lanes per group and
+// 64 / LPG groups per wave, one 4-wide access per lane.
+template <typename TG, typename TO, int LPG>
+__global__ __launch_bounds__(256) void gated_group_rmsnorm_narrow_kernel(
+    const float* __restrict__ y, const TG* __restrict__ gate_src,
+    const int64_t gld, const int gcol0, const float* __restrict__ w,
+    TO* __restrict__ out, const int64_t old, const int N, const int groups,
+    const float eps, const bool gate_silu, const bool gate_first) {
+  const int64_t row = blockIdx.y;
+  const int grp = (blockIdx.x * blockDim.x + threadIdx.x) / LPG;
+  const int gs = N / groups, e = (threadIdx.x % LPG) * 4;
+  const bool on = grp < groups && e < gs;
+  const int64_t c = (int64_t)grp * gs + e;
+  vecf<4> v, g;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v.v[j] = g.v[j] = 0.f;
+  if (on) {
+    v = ldw<4, float>(y + row * N + c);
+    g = ldw<4, TG>(gate_src + row * gld + gcol0 + c);
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    g.v[j] = gate_silu ? g.v[j] * sigmoid_f(g.v[j]) : sigmoid_f(g.v[j]);
+    if (gate_first) v.v[j] *= g.v[j];
+    ss += v.v[j] * v.v[j];
+  }
+#pragma unroll
+  for (int off = LPG / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+  if (!on) return;
+  const float r = 1.0f / sqrtf(ss / (float)gs + eps);
+  const vecf<4> wv = ldw<4, float>(w + c);
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    v.v[j] = v.v[j] * r * wv.v[j];
+    if (!gate_first) v.v[j] *= g.v[j];
+  }
+  stw<4, TO>(out + row * old + c, v);
+}
+
 // Wide groups (>= 1024 channels): one workgroup per (row, group), 4-wide
 // accesses when the group size and the gate's stride and offset allow.
 template <typename TG, typename TO, int W>
@@ -777,7 +817,12 @@ void gated_group_rmsnorm(torch::Tensor y, torch::Tensor gate_src,
   const bool v4 = gs % 4 == 0 && gate_src.size(1) % 4 == 0 &&
                   gate_col0 % 4 == 0 && out.stride(0) % 4 == 0 &&
                   out.storage_offset() % 4 == 0;
-  const dim3 grid(wide ? (unsigned)groups : (unsigned)((groups + 3) / 4),
+  // lanes per group of the narrow kernel
+  const int lpg = v4 && gs <= 32 ? 8 : gs <= 64 ? 16 : gs <= 128 ? 32 : 64;
+  const bool narrow = v4 && gs <= 256;
+  const dim3 grid(wide ? (unsigned)groups
+                  : narrow ? (unsigned)((groups * (int64_t)lpg + 255) / 256)
+                           : (unsigned)((groups + 3) / 4),
                   (unsigned)M);
 #define GG_ARGS(TG, TO)                                                      \
   grid, dim3(256), 0, st, y.data_ptr<float>(),                               \
@@ -791,6 +836,18 @@ void gated_group_rmsnorm(torch::Tensor y, torch::Tensor gate_src,
                          GG_ARGS(TG, TO));                                   \
     else if (wide)                                                           \
       hipLaunchKernelGGL((gated_group_rmsnorm_wide_kernel<TG, TO, 1>),       \
+                         GG_ARGS(TG, TO));                                   \
+    else if (narrow && lpg == 8)                                             \
+      hipLaunchKernelGGL((gated_group_rmsnorm_narrow_kernel<TG, TO, 8>),     \
+                         GG_ARGS(TG, TO));                                   \
+    else if (narrow && lpg == 16)                                            \
+      hipLaunchKernelGGL((gated_group_rmsnorm_narrow_kernel<TG, TO, 16>),    \
+                         GG_ARGS(TG, TO));                                   \
+    else if (narrow && lpg == 32)                                            \
+      hipLaunchKernelGGL((gated_group_rmsnorm_narrow_kernel<TG, TO, 32>),    \
+                         GG_ARGS(TG, TO));                                   \
+    else if (narrow)                                                         \
+      hipLaunchKernelGGL((gated_group_rmsnorm_narrow_kernel<TG, TO, 64>),    \
                          GG_ARGS(TG, TO));                                   \
     else                                                                     \
       hipLaunchKernelGGL((gated_group_rmsnorm_kernel<TG, TO>),               \

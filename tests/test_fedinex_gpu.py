@@ -199,6 +199,59 @@ def test_mlstm_scan(dt, H, d, dv, T, ib, fb):
 
 
 @pytest.mark.parametrize("dt", DTS)
+@pytest.mark.parametrize("kind", ["gla", "mlstm"])
+@pytest.mark.parametrize("H,d,dv", [(3, 64, 32), (2, 20, 70), (1, 1, 1),
+                                    (4, 128, 128), (2, 130, 200),
+                                    (1, 300, 65), (2, 9, 1100), (2, 24, 1028),
+                                    (5, 16, 9)])
+def test_recurrent_heads(dt, kind, H, d, dv):
+    """A portion (scan and norm), then decode steps (one fused launch) with an
+    idle row and a row that starts: results, written into a column range, and
+    states against the reference."""
+    torch.manual_seed(H * d + dv)
+    B, Bc, T, rank = 4, 5, 3, 7
+    q0, k0, v0 = 3, 3 + H * d, 3 + 2 * H * d
+    g0 = v0 + H * dv + 1
+    e0 = g0 + H * dv + 3
+    ld = e0 + max(rank, 2 * H) + 2
+    w = 1 + 0.2 * torch.randn(H * dv, device=DEV)
+    nt = ops.scan_tiles(d, dv)
+    S = torch.randn(Bc, H, d, dv, device=DEV)
+    n_ = torch.randn(Bc, H, 1, d, device=DEV).repeat(1, 1, nt, 1).contiguous()
+    m = torch.rand(Bc, H, 1, device=DEV).repeat(1, 1, nt).contiguous()
+    if kind == "gla":
+        par = [torch.randn(rank, H * d, device=DEV) * rank ** -0.5,
+               torch.randn(H * d, device=DEV) + 1]
+        cols, const, states = (q0, k0, v0, e0), (0.25, d ** -0.5), [S]
+    else:
+        par = [torch.randn(H, device=DEV), torch.randn(H, device=DEV) + 1]
+        cols, const = (q0, k0, v0, e0, e0 + H), (10.0, d ** -0.5)
+        states = [S, n_, m]
+    cpu_states = [t.cpu().clone() for t in states]
+    act = "silu" if kind == "gla" else "sigmoid"
+    fn = getattr(ops, kind + "_heads")
+    pos, lens = _i32([40, 0, 7, 0]), _i32([T, 2, 0, 0])
+    slots = _i32([3, 0, 1, 4])
+    for step in range(4):
+        n = T if step == 0 else 1
+        src = torch.randn(B * n, ld, device=DEV).to(dt)
+        buf = torch.full((B * n, H * dv + 8), 7.0, device=DEV).to(dt)
+        fn(src, *cols, *par, *const, *states, pos.to(DEV), n, lens.to(DEV),
+           slots.to(DEV), w, g0, act, 1e-5, out=buf[:, 4:4 + H * dv])
+        want = fn(src.cpu(), *cols, *[p.cpu() for p in par], *const,
+                  *cpu_states, pos, n, lens, slots, w.cpu(), g0, act, 1e-5)
+        tol = _tol(dt) if dt == torch.bfloat16 else dict(atol=3e-3, rtol=3e-3)
+        torch.testing.assert_close(buf[:, 4:4 + H * dv].cpu().float(),
+                                   want.float(), **tol)
+        assert bool((buf[:, :4] == 7).all()) and \
+            bool((buf[:, 4 + H * dv:] == 7).all())
+        for a, b in zip(states, cpu_states):
+            torch.testing.assert_close(a.cpu(), b, atol=2e-4, rtol=2e-4)
+        pos = (pos + lens).to(torch.int32)
+        lens = _i32([1, 1, 0, 1])
+
+
+@pytest.mark.parametrize("dt", DTS)
 @pytest.mark.parametrize("I", [64, 36, 1030, 7])
 def test_clamped_act(dt, I):
     torch.manual_seed(I)
@@ -263,7 +316,9 @@ def test_clamped_expert_rows(T, W, I, E, top):
 
 
 @pytest.mark.parametrize("odt", DTS)
-@pytest.mark.parametrize("N,groups", [(96, 3), (64, 64), (2048, 2), (30, 5)])
+@pytest.mark.parametrize("N,groups", [(96, 3), (64, 64), (2048, 2), (30, 5),
+                                      (64, 2), (280, 5), (128, 2), (1024, 4),
+                                      (640, 5)])
 def test_grouped_norm_into_columns(odt, N, groups):
     torch.manual_seed(N)
     M = 5
