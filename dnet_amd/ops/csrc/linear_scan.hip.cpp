@@ -14,15 +14,30 @@
 // states and results are fp32 whatever the activation dtype ("short" stands
 // for bf16 bits).
 //
-// Layout: a workgroup owns a tile of JB value columns of one head of one batch
-// row and walks the tokens in order; thread (column j, slice s) keeps rows
+// Prompts (linear_chunk_kernel): a workgroup owns a tile of value columns of one
+// head of one batch row and walks the tokens in chunks of 16. With w_s(t) = the
+// key of token s carried to token t (k_s times every decay after s up to t),
+// a chunk is
+//     A[t][s] = q_t . w_s(t)  (s <= t)
+//     O = A V + (q_t times the chunk's decays up to t) S
+//     S <- (all the chunk's decays) S + w_s(last)^T V
+// A comes from walking w token by token in registers (products of decays only,
+// never a quotient, so that strong decays underflow instead of overflowing);
+// the matrix products run on v_mfma_f32_16x16x4_f32 (fp32 operands: the state,
+// the decays and what they multiply stay 32-bit), the state tile stays in the
+// accumulator fragments. The next chunk's rows are in flight meanwhile.
+// The matrix memory's normalizer n and maximum m ride along; every 64 value
+// columns have their own copy of both in the state, so that no workgroup reads
+// what another one writes.
+//
+// The decays of gated linear attention are formed for all tokens at once by a
+// kernel in front (low_rank_decay_kernel).
+//
+// Key sizes above 256 (and low-rank inputs above 1024) take linear_scan_kernel,
+// a walk over the tokens one by one: thread (column j, slice s) keeps rows
 // [R s, R s + R) of column j in registers, the slices of a column are
-// neighbouring lanes. Tokens are staged through LDS in chunks, with every
-// gate evaluated once per chunk; the chunk's results are gathered in LDS and
-// written out as rows. The matrix memory's normalizer n is one more column
-// (of ones) on a wave of its own, which also forms the gates and the running
-// maximum; every column tile keeps its own copy of n and m, so that no
-// workgroup reads what another one writes.
+// neighbouring lanes, tokens are staged through LDS in chunks with every gate
+// evaluated once, and n is one more column (of ones) on a wave of its own.
 //
 // Decode steps (one token per row) have a kernel of their own: a workgroup owns
 // a head of a batch row, streams its state once through 16 B accesses, and goes
@@ -45,6 +60,13 @@ __device__ __forceinline__ float log_sigmoid(float z) {
   return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
 }
 
+// sigmoid(z)^p; the hardware exponential and logarithm are within a few 1e-7 of
+// the decay here (the logarithm's argument lies in [1, 2])
+__device__ __forceinline__ float decay_of(float z, float p) {
+  const float ls = fminf(z, 0.f) - __logf(1.f + __expf(-fabsf(z)));
+  return __expf(ls * p);
+}
+
 constexpr int kGla = 0, kMlstm = 1;
 constexpr float kDenEps = 1e-6f;
 
@@ -58,6 +80,7 @@ struct ScanArgs {
   // gla: low-rank input at column a0, a2t [rank][H*d], bias [H*d]
   const float* a2t;
   const float* ab;
+  const float* alpha;        // prompts: the decays, [B*T, H*d]
   // mlstm: gate columns i0, f0 with biases, n [Bc, H, NT, d], m [Bc, H, NT]
   const float* ib;
   const float* fb;
@@ -193,7 +216,7 @@ __global__ __launch_bounds__(1024) void linear_scan_kernel(const ScanArgs a) {
         for (int u = 0; u < 4; ++u)
           if (tg + u < tc)
             sA[(tg + u) * DP + at] =
-                i < d ? expf(log_sigmoid(z[u]) * a.inv_tau) : 0.f;
+                i < d ? decay_of(z[u], a.inv_tau) : 0.f;
       }
       __syncthreads();
     }
@@ -257,6 +280,448 @@ __global__ __launch_bounds__(1024) void linear_scan_kernel(const ScanArgs a) {
     }
   }
   if (ncol && lane == 0) *mp = m;
+}
+
+// ---- prompts in chunks on the matrix cores -------------------------------------
+using f32x4 = __attribute__((ext_vector_type(4))) float;
+
+// sum over the 16 lanes of a row, in every lane
+template <int CTRL> __device__ __forceinline__ float row_rot(float x) {
+  union { float f; int i; } u;
+  u.f = x;
+  u.i = __builtin_amdgcn_update_dpp(0, u.i, CTRL, 0xf, 0xf, true);
+  return u.f;
+}
+__device__ __forceinline__ float row16_sum(float x) {
+  x += row_rot<0x128>(x);                   // row_ror:8, 4, 2, 1
+  x += row_rot<0x124>(x);
+  x += row_rot<0x122>(x);
+  x += row_rot<0x121>(x);
+  return x;
+}
+
+// x times the values of the lower lanes of its row of 16 (inclusive product)
+template <int CTRL> __device__ __forceinline__ float row_shift1(float x) {
+  union { float f; int i; } u, one;
+  u.f = x;
+  one.f = 1.f;                              // lanes without a source
+  u.i = __builtin_amdgcn_update_dpp(one.i, u.i, CTRL, 0xf, 0xf, false);
+  return u.f;
+}
+__device__ __forceinline__ float row16_prod_upto(float x) {
+  x *= row_shift1<0x111>(x);                // row_shr:1, 2, 4, 8
+  x *= row_shift1<0x112>(x);
+  x *= row_shift1<0x114>(x);
+  x *= row_shift1<0x118>(x);
+  return x;
+}
+__device__ __forceinline__ float from_lane(float x, int l) {
+  union { float f; int i; } u;
+  u.f = x;
+  u.i = __builtin_amdgcn_readlane(u.i, l);
+  return u.f;
+}
+
+constexpr int kTok = 16;                    // tokens of a chunk
+constexpr int kAP = 20;                     // LDS pitch of a row of A
+
+// LDS floats of a chunk kernel with DPAD key rows and JB columns
+__host__ __device__ constexpr int chunk_lds(int kind, int DPAD, int JB) {
+  return kTok * (DPAD + 4) * (kind == kGla ? 3 : 2) + kTok * (JB + 4) +
+         kTok * kAP + DPAD + (kind == kGla ? 4 * DPAD : 9 * kTok);
+}
+
+// decays of a prompt's tokens: grid (channel tiles, token tiles), a thread walks
+// 16 tokens of one channel, every weight read once for them
+template <typename T>
+__global__ __launch_bounds__(256) void low_rank_decay_kernel(
+    const ScanArgs a, float* __restrict__ alpha, const int64_t M) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];   // [rank][16]
+  const int64_t m0 = (int64_t)blockIdx.y * kTok;
+  const int mt = (int)min((int64_t)kTok, M - m0);
+  const int HD = a.H * a.d, c = blockIdx.x * 256 + threadIdx.x;
+  const T* src = reinterpret_cast<const T*>(a.src);
+  for (int idx = threadIdx.x; idx < kTok * a.rank; idx += 256) {
+    const int tt = idx / a.rank, r = idx % a.rank;
+    sm[r * kTok + tt] = ldx<T>(src + (m0 + min(tt, mt - 1)) * a.ld + a.a0 + r);
+  }
+  __syncthreads();
+  if (c >= HD) return;
+  float z[kTok];
+  const float ab = a.ab[c];
+#pragma unroll
+  for (int t = 0; t < kTok; ++t) z[t] = ab;
+#pragma unroll 4
+  for (int r = 0; r < a.rank; ++r) {
+    const float w = a.a2t[(int64_t)r * HD + c];
+#pragma unroll
+    for (int q = 0; q < kTok / 4; ++q) {
+      const float4 x = *reinterpret_cast<const float4*>(sm + r * kTok + q * 4);
+      z[4 * q + 0] = fmaf(w, x.x, z[4 * q + 0]);
+      z[4 * q + 1] = fmaf(w, x.y, z[4 * q + 1]);
+      z[4 * q + 2] = fmaf(w, x.z, z[4 * q + 2]);
+      z[4 * q + 3] = fmaf(w, x.w, z[4 * q + 3]);
+    }
+  }
+#pragma unroll
+  for (int t = 0; t < kTok; ++t)
+    if (t < mt) alpha[(m0 + t) * HD + c] = decay_of(z[t], a.inv_tau);
+}
+
+// grid (H * column blocks, B), 4 waves of CF x 16 columns; the matrix memory has
+// a fifth wave that forms the next chunk's gates and running maximum while the
+// others work on the current one. M4 = key rows / 64. Fragments of
+// v_mfma_f32_16x16x4_f32: lane (c = lane & 15, hi = lane >> 4) holds A[c][hi],
+// B[hi][c] and rows hi*4 + r of column c of the result. The sum over k may run
+// in any order: step r takes rows hi*4 + r, which are what a lane's state
+// fragment holds in register r, and one 16 B read of an A row.
+template <typename T, int M4, int CF, int KIND>
+__global__ __launch_bounds__(M4 == 4 && KIND == kGla ? 256 : 320)
+void linear_chunk_kernel(const ScanArgs a) {
+  constexpr int DPAD = M4 * 64, DF = M4 * 4, DP = DPAD + 4;
+  constexpr int JB = 64 * CF, VP = JB + 4;
+  constexpr int QN = kTok * DPAD / 256, VN = kTok * JB / 256;
+  const int NB = (a.dv + JB - 1) / JB;      // column blocks
+  const int h = blockIdx.x / NB, blk = blockIdx.x % NB, b = blockIdx.y;
+  const int n = a.lens ? min(a.lens[b], a.T) : a.T;
+  const int slot = a.slots ? a.slots[b] : b;
+  const int p0 = a.pos[b];
+  if (n <= 0 || slot < 0 || slot >= a.Bc || p0 < 0) return;   // uniform
+  const int d = a.d, dv = a.dv, j0 = blk * JB, tid = threadIdx.x;
+  const int wave = tid >> 6, lane = tid & 63, c16 = lane & 15, hi = lane >> 4;
+  const bool work = wave < 4;               // else: the gates' wave
+
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  float* sQ = sm;                           // [16][DP]
+  float* sK = sQ + kTok * DP;               // [16][DP]
+  float* sAl = sK + kTok * DP;              // gla: decays [16][DP]
+  float* sV = sAl + (KIND == kGla ? kTok * DP : 0);   // [16][VP]
+  float* sAm = sV + kTok * VP;              // [16][kAP]
+  float* sE = sAm + kTok * kAP;             // gla: the chunk's decays; mlstm: n
+  float* sGp = sE + DPAD;                   // gla: decays of 4 tokens [4][DPAD]
+  float* sGate = sE + DPAD;                 // mlstm: 2 x (keep, put, e^-m, keeps
+                                            // up to t) [16]
+  float* sDen = sGate + 8 * kTok;           // mlstm: 1 / denominator [16]
+
+  f32x4 S[CF][DF];
+  float* sp = a.state + (((int64_t)slot * a.H + h) * d) * dv;
+#pragma unroll
+  for (int f = 0; f < CF; ++f) {
+    const int j = j0 + (wave * CF + f) * 16 + c16;
+#pragma unroll
+    for (int g = 0; g < DF; ++g)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int row = g * 16 + hi * 4 + r;
+        S[f][g][r] = work && p0 > 0 && row < d && j < dv
+                         ? sp[(int64_t)row * dv + j] : 0.f;
+      }
+  }
+  // copies of n and m that belong to this block
+  const int tile0 = blk * CF, tile1 = min(tile0 + CF, a.NT);
+  float m = 0.f, ib = 0.f, fb = 0.f;
+  const int ci = tid % DPAD;                // a thread's channel when staging
+  if constexpr (KIND == kMlstm) {
+    const float* np = a.nst + (((int64_t)slot * a.H + h) * a.NT + tile0) * d;
+    if (work)
+      for (int i = tid; i < DPAD; i += 256)
+        sE[i] = p0 > 0 && i < d ? np[i] : 0.f;
+    if (p0 > 0) m = a.mst[((int64_t)slot * a.H + h) * a.NT + tile0];
+    ib = a.ib[h];
+    fb = a.fb[h];
+  }
+
+  // The next chunk's projection values travel into registers: loads without
+  // conditions (out-of-range ones repeat a valid element and are dropped where
+  // they are stored to LDS).
+  const T* src = reinterpret_cast<const T*>(a.src) + (int64_t)b * a.T * a.ld;
+  T rq[QN], rk[QN], rv[VN];
+  float ra[M4][4];                          // gla: decays of four tokens
+  const int qc = h * d + min(ci, d - 1);
+  const int vcol = tid % JB, vc = h * dv + min(j0 + vcol, dv - 1);
+  const int ldi = (int)a.ld;
+  auto fetch = [&](const int t0) {
+    const int last = min(kTok, n - t0) - 1;
+    const T* row = src + (int64_t)t0 * a.ld;
+    const T* q = row + a.q0 + qc;
+    const T* k = row + a.k0 + qc;
+    const T* v = row + a.v0 + vc;
+#pragma unroll
+    for (int u = 0; u < QN; ++u) {
+      const int at = min((tid + u * 256) / DPAD, last) * ldi;
+      rq[u] = q[at];
+      rk[u] = k[at];
+    }
+#pragma unroll
+    for (int u = 0; u < VN; ++u)
+      rv[u] = v[min((tid + u * 256) / JB, last) * ldi];
+    if constexpr (KIND == kGla) {
+      const float* al = a.alpha + ((int64_t)b * a.T + t0) * a.H * d + qc;
+#pragma unroll
+      for (int u0 = 0; u0 < M4; ++u0)
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          ra[u0][u] = al[min(((tid + u0 * 256) / DPAD) * 4 + u, last) *
+                         (a.H * d)];
+    }
+  };
+  // gates of the chunk at t0 into buffer buf (mlstm, the fifth wave)
+  auto gates = [&](const int t0, float* g) {
+    const int tc = min(kTok, n - t0);
+    const T* sr = src + (int64_t)(t0 + min(lane, tc - 1)) * a.ld + h;
+    const float gi = ldx<T>(sr + a.i0), gf = ldx<T>(sr + a.f0);
+    const float li = a.cap * tanhf((gi + ib) / a.cap);
+    const float lf = log_sigmoid(a.cap * tanhf((gf + fb) / a.cap));
+    float before = 0.f, after = 0.f;
+#pragma unroll
+    for (int t = 0; t < kTok; ++t) {        // the running maximum, in order
+      const float f = from_lane(lf, t), i = from_lane(li, t);
+      const float mn = fmaxf(f + m, i);
+      if (lane == t) {
+        before = f + m;
+        after = mn;
+      }
+      if (t < tc) m = mn;
+    }
+    const bool real = lane < tc;            // neutral tokens behind the last
+    const float keep = real ? expf(before - after) : 1.f;
+    const float prod = row16_prod_upto(keep);
+    if (lane < kTok) {
+      g[lane] = keep;
+      g[kTok + lane] = real ? expf(li - after) : 0.f;
+      g[2 * kTok + lane] = expf(-after);
+      g[3 * kTok + lane] = prod;
+    }
+  };
+  if (work) fetch(0);
+  else gates(0, sGate);
+
+  int buf = 0;
+  for (int t0 = 0; t0 < n; t0 += kTok, buf ^= 1) {
+    const int tc = min(kTok, n - t0);
+    const float* sKeep = sGate + buf * 4 * kTok;
+    const float* sPut = sKeep + kTok;
+    const float* sEm = sPut + kTok;
+    const float* sP = sEm + kTok;           // products of keep up to t
+    float al[M4][4];                        // gla: own decays
+    __syncthreads();                        // previous chunk consumed
+    if (work) {
+#pragma unroll
+      for (int u = 0; u < QN; ++u) {
+        const int tt = (tid + u * 256) / DPAD, at = tt * DP + ci;
+        const bool in = tt < tc && ci < d;
+        sQ[at] = in ? ldx<T>(&rq[u]) * a.qscale : 0.f;
+        sK[at] = in ? ldx<T>(&rk[u]) : 0.f;
+      }
+#pragma unroll
+      for (int u = 0; u < VN; ++u) {
+        const int tt = (tid + u * 256) / JB;
+        sV[tt * VP + vcol] =
+            tt < tc && j0 + vcol < dv ? ldx<T>(&rv[u]) : 0.f;
+      }
+      if constexpr (KIND == kGla) {
+#pragma unroll
+        for (int u0 = 0; u0 < M4; ++u0) {
+          const int tg = ((tid + u0 * 256) / DPAD) * 4;
+          float p = 1.f;
+#pragma unroll
+          for (int u = 0; u < 4; ++u) {
+            al[u0][u] = tg + u < tc ? ra[u0][u] : 1.f;
+            sAl[(tg + u) * DP + ci] = al[u0][u];
+            p *= al[u0][u];
+          }
+          sGp[(tg / 4) * DPAD + ci] = p;
+        }
+      }
+    }
+    __syncthreads();
+    if (work && t0 + kTok < n) fetch(t0 + kTok);
+    if (work) {
+      // A, and the keys carried to the chunk's end: 16 lanes per key s, four
+      // channels of every 64 per lane; lane sl keeps A[sl][s]
+      const int s = tid >> 4, sl = tid & 15;
+      float4 k4[M4], w4[M4];
+      const float put = KIND == kMlstm ? sPut[s] : 1.f;
+      float carried = 0.f, mine = 0.f;      // mlstm: the key's scalar factor
+#pragma unroll
+      for (int q = 0; q < M4; ++q) {
+        k4[q] = *reinterpret_cast<const float4*>(sK + s * DP + q * 64 + sl * 4);
+        w4[q] = make_float4(0.f, 0.f, 0.f, 0.f);
+      }
+#pragma unroll 1
+      for (int tg = 0; tg < kTok; tg += 4) {
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          const int t = tg + u;
+          const bool own = t == s;
+          float acc = 0.f;
+#pragma unroll
+          for (int q = 0; q < M4; ++q) {
+            const int at = t * DP + q * 64 + sl * 4;
+            const float4 qv = *reinterpret_cast<const float4*>(sQ + at);
+            float4 w = k4[q];
+            if constexpr (KIND == kGla) {
+              const float4 av = *reinterpret_cast<const float4*>(sAl + at);
+              w.x = own ? k4[q].x : w4[q].x * av.x;
+              w.y = own ? k4[q].y : w4[q].y * av.y;
+              w.z = own ? k4[q].z : w4[q].z * av.z;
+              w.w = own ? k4[q].w : w4[q].w * av.w;
+              w4[q] = w;
+            }
+            acc = fmaf(qv.x, w.x, acc);
+            acc = fmaf(qv.y, w.y, acc);
+            acc = fmaf(qv.z, w.z, acc);
+            acc = fmaf(qv.w, w.w, acc);
+          }
+          if constexpr (KIND == kMlstm) {
+            carried = own ? put : carried * sKeep[t];
+            acc *= carried;
+          }
+          acc = row16_sum(acc);
+          if (sl == t) mine = acc;
+        }
+      }
+      sAm[sl * kAP + s] = mine;
+#pragma unroll
+      for (int q = 0; q < M4; ++q) {
+        if constexpr (KIND == kMlstm)
+          w4[q] = make_float4(k4[q].x * carried, k4[q].y * carried,
+                              k4[q].z * carried, k4[q].w * carried);
+        *reinterpret_cast<float4*>(sK + s * DP + q * 64 + sl * 4) = w4[q];
+      }
+    } else if (t0 + kTok < n) {
+      gates(t0 + kTok, sGate + (buf ^ 1) * 4 * kTok);
+    }
+    __syncthreads();
+    if constexpr (KIND == kGla) {
+      // queries times the decays up to them; the whole chunk's decays
+#pragma unroll
+      for (int u0 = 0; u0 < M4; ++u0) {
+        const int g = (tid + u0 * 256) / DPAD;
+        const float g0 = sGp[ci], g1 = sGp[DPAD + ci], g2 = sGp[2 * DPAD + ci];
+        float p = (g > 0 ? g0 : 1.f) * (g > 1 ? g1 : 1.f) * (g > 2 ? g2 : 1.f);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          p *= al[u0][u];
+          sQ[(g * 4 + u) * DP + ci] *= p;
+        }
+        if (g == 3) sE[ci] = p;
+      }
+    } else if (work) {
+      // n . q of every token: 16 lanes per token
+      const int t = tid >> 4, l = tid & 15;
+      const float at = sAm[t * kAP + l];
+      float nq = 0.f;
+#pragma unroll
+      for (int q = 0; q < M4; ++q) {
+        const float4 qv =
+            *reinterpret_cast<const float4*>(sQ + t * DP + q * 64 + l * 4);
+        const float4 nv = *reinterpret_cast<const float4*>(sE + q * 64 + l * 4);
+        nq = fmaf(qv.x, nv.x, nq);
+        nq = fmaf(qv.y, nv.y, nq);
+        nq = fmaf(qv.z, nv.z, nq);
+        nq = fmaf(qv.w, nv.w, nq);
+      }
+      nq = row16_sum(fmaf(nq, sP[t], at));  // (A is zero above the diagonal)
+      if (l == 0) sDen[t] = 1.f / (fmaxf(fabsf(nq), sEm[t]) + kDenEps);
+    }
+    __syncthreads();
+    if (work) {
+      const float pq = KIND == kMlstm ? sP[c16] : 1.f;
+      const float pc = KIND == kMlstm ? sP[kTok - 1] : 1.f;
+      // A row c16, entries hi*4 .. +3
+      const float4 a4 =
+          *reinterpret_cast<const float4*>(sAm + c16 * kAP + hi * 4);
+      const float am[4] = {a4.x, a4.y, a4.z, a4.w};
+      float bv[CF][4];
+      f32x4 o[CF];
+#pragma unroll
+      for (int f = 0; f < CF; ++f) {
+        o[f] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          bv[f][r] = sV[(hi * 4 + r) * VP + (wave * CF + f) * 16 + c16];
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+#pragma unroll
+        for (int f = 0; f < CF; ++f)
+          o[f] = __builtin_amdgcn_mfma_f32_16x16x4f32(am[r], bv[f][r], o[f], 0,
+                                                      0, 0);
+#pragma unroll
+      for (int g = 0; g < DF; ++g) {
+        const float4 q4 =
+            *reinterpret_cast<const float4*>(sQ + c16 * DP + g * 16 + hi * 4);
+        const float qr[4] = {q4.x * pq, q4.y * pq, q4.z * pq, q4.w * pq};
+        float e[4] = {pc, pc, pc, pc};
+        if constexpr (KIND == kGla) {
+          const float4 e4 =
+              *reinterpret_cast<const float4*>(sE + g * 16 + hi * 4);
+          e[0] = e4.x; e[1] = e4.y; e[2] = e4.z; e[3] = e4.w;
+        }
+        float ka[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          ka[r] = sK[(hi * 4 + r) * DP + g * 16 + c16];
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+          for (int f = 0; f < CF; ++f)
+            o[f] = __builtin_amdgcn_mfma_f32_16x16x4f32(qr[r], S[f][g][r], o[f],
+                                                        0, 0, 0);
+#pragma unroll
+        for (int f = 0; f < CF; ++f) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) S[f][g][r] *= e[r];
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            S[f][g] = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[r], bv[f][r],
+                                                           S[f][g], 0, 0, 0);
+        }
+      }
+#pragma unroll
+      for (int f = 0; f < CF; ++f) {
+        const int j = j0 + (wave * CF + f) * 16 + c16;
+        float* op = a.o + ((int64_t)b * a.T + t0 + hi * 4) * a.H * dv + h * dv + j;
+        float4 den = make_float4(1.f, 1.f, 1.f, 1.f);
+        if constexpr (KIND == kMlstm)
+          den = *reinterpret_cast<const float4*>(sDen + hi * 4);
+        const float dn[4] = {den.x, den.y, den.z, den.w};
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (hi * 4 + r < tc && j < dv)
+            op[(int64_t)r * a.H * dv] =
+                KIND == kMlstm ? o[f][r] * dn[r] : o[f][r];
+      }
+      if constexpr (KIND == kMlstm)         // n was last read before the barrier
+        for (int i = tid; i < DPAD; i += 256) {
+          float v = sE[i] * pc;
+#pragma unroll
+          for (int t = 0; t < kTok; ++t) v += sK[t * DP + i];
+          sE[i] = v;
+        }
+    }
+  }
+#pragma unroll
+  for (int f = 0; f < CF; ++f) {
+    const int j = j0 + (wave * CF + f) * 16 + c16;
+#pragma unroll
+    for (int g = 0; g < DF; ++g)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int row = g * 16 + hi * 4 + r;
+        if (work && row < d && j < dv) sp[(int64_t)row * dv + j] = S[f][g][r];
+      }
+  }
+  if constexpr (KIND == kMlstm) {
+    for (int tile = tile0; tile < tile1; ++tile) {
+      float* np = a.nst + (((int64_t)slot * a.H + h) * a.NT + tile) * d;
+      if (work)
+        for (int i = tid; i < d; i += 256) np[i] = sE[i];   // own elements
+      else if (lane == 0)
+        a.mst[((int64_t)slot * a.H + h) * a.NT + tile] = m;
+    }
+  }
 }
 
 // ---- one decode step -----------------------------------------------------------
@@ -355,7 +820,7 @@ __global__ __launch_bounds__(256) void linear_step_kernel(const ScanArgs a,
 #pragma unroll 16
       for (int r = 0; r < a.rank; ++r)
         z = fmaf(wp[(int64_t)r * a.H * d], ldx<T>(src + a.a0 + r), z);
-      sA[i] = expf(log_sigmoid(z) * a.inv_tau);
+      sA[i] = decay_of(z, a.inv_tau);
     } else {
       // the normalizer, every column tile's copy
       float* np = a.nst + ((int64_t)slot * a.H + h) * a.NT * d + i;
@@ -480,6 +945,47 @@ void scan_launch(ScanArgs& a, int kind, const torch::Tensor& src,
                  o.size(1) == H * dv, "o fp32 [B*T, H*dv]");
   if (M == 0) return;
   a.o = o.data_ptr<float>();
+  auto st = current_stream();
+  // the copies of n and m belong to 64 columns each there
+  const bool tiles64 = NT == (dv + 63) / 64;
+  const int M4 = d <= 64 ? 1 : (d <= 128 ? 2 : 4);
+  // two column fragments per wave when that still fills the chip
+  const int CF = dv > 64 && M4 < 4 && H * B * ((dv + 127) / 128) >= 256 ? 2 : 1;
+  const size_t clds =
+      (size_t)chunk_lds(kind, M4 * 64, 64 * CF) * sizeof(float);
+  const size_t dlds = (size_t)kTok * a.rank * sizeof(float);
+  if (d <= 256 && tiles64 && clds <= 64 * 1024 && dlds <= 64 * 1024) {
+    torch::Tensor alpha;
+    if (kind == kGla) {
+      alpha = torch::empty({M, H * d}, o.options());
+      a.alpha = alpha.data_ptr<float>();
+      const dim3 dgrid((unsigned)((H * d + 255) / 256),
+                       (unsigned)((M + kTok - 1) / kTok));
+      if (is_bf16(src))
+        hipLaunchKernelGGL((low_rank_decay_kernel<short>), dgrid, dim3(256),
+                           dlds, st, a, alpha.data_ptr<float>(), M);
+      else
+        hipLaunchKernelGGL((low_rank_decay_kernel<float>), dgrid, dim3(256),
+                           dlds, st, a, alpha.data_ptr<float>(), M);
+    }
+    const dim3 cgrid((unsigned)(H * ((dv + 64 * CF - 1) / (64 * CF))),
+                     (unsigned)B);
+#define LC(TT, MM, CC, KK)                                                    \
+  hipLaunchKernelGGL((linear_chunk_kernel<TT, MM, CC, KK>), cgrid,            \
+                     dim3(KK == kMlstm ? 320 : 256), clds, st, a)
+#define LC_M(TT, KK)                                                          \
+  do {                                                                        \
+    if (M4 == 4) LC(TT, 4, 1, KK);                                            \
+    else if (M4 == 2) { if (CF == 2) LC(TT, 2, 2, KK); else LC(TT, 2, 1, KK); } \
+    else { if (CF == 2) LC(TT, 1, 2, KK); else LC(TT, 1, 1, KK); }            \
+  } while (0)
+#define LC_K(TT) do { if (kind == kGla) LC_M(TT, kGla); else LC_M(TT, kMlstm); } while (0)
+    if (is_bf16(src)) LC_K(short); else LC_K(float);
+#undef LC_K
+#undef LC_M
+#undef LC
+    return;
+  }
   const int R = d <= 32 ? 8 : (d <= 128 ? 16 : 32);
   a.NS = 1;
   while (a.NS * R < d) a.NS *= 2;           // power of two, <= 16
@@ -498,7 +1004,6 @@ void scan_launch(ScanArgs& a, int kind, const torch::Tensor& src,
   const size_t lds = floats(a.TC) * sizeof(float);
   DNET_CHECK(lds <= 64 * 1024, "linear_scan: sizes exceed LDS");
   const dim3 grid((unsigned)(H * NT), (unsigned)B);
-  auto st = current_stream();
 #define LS(TT, RR, KK)                                                        \
   hipLaunchKernelGGL((linear_scan_kernel<TT, RR, KK>), grid, dim3(threads),   \
                      lds, st, a)
