@@ -290,3 +290,36 @@ def test_shared_rows_family_over_two_shards(cluster):
         assert texts[0] == texts[1]
         r = c.post(f"{api}/v1/unload_model")
         assert r.status_code == 200
+
+
+@pytest.mark.timeout(300)
+def test_value_mixing_family_over_two_shards(cluster):
+    """A family whose attention layers mix in the values of the first one
+    (fedinex), split so that a reader sits on the other shard: the step's
+    values ride the hops, chats complete and repeat, also when the slot is
+    used again."""
+    api = cluster["api"]
+    name = "fedinex-tiny-random"
+    with httpx.Client(timeout=180) as c:
+        r = c.post(f"{api}/v1/prepare_topology_manual", json={
+            "model": name,
+            "assignments": [
+                {"instance": "shard0", "layers": [0]},
+                {"instance": "shard1", "layers": [1, 2, 3]}]})
+        assert r.status_code == 200, r.text
+        r = c.post(f"{api}/v1/load_model",
+                   json={"model": name, "max_tokens": 8})
+        assert r.status_code == 200, r.text
+        texts = []
+        for _ in range(2):          # greedy: the same prompt repeats exactly
+            r = c.post(f"{api}/v1/chat/completions", json={
+                "model": name, "stream": False, "max_tokens": 8,
+                "temperature": 0.0,
+                "messages": [{"role": "user", "content": "values please"}]})
+            assert r.status_code == 200, r.text
+            body = r.json()
+            assert body["usage"]["completion_tokens"] >= 1
+            texts.append(body["choices"][0]["message"]["content"])
+        assert texts[0] == texts[1]
+        r = c.post(f"{api}/v1/unload_model")
+        assert r.status_code == 200
