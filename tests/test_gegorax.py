@@ -794,7 +794,7 @@ def _ring_rank_main(rank, world, port, q):
     dist.init_process_group("gloo", rank=rank, world_size=world)
     out = _ring_run(rank, world)
     if rank == 0:
-        q.put(out)
+        q.put(out.tolist())
     dist.destroy_process_group()
 
 
@@ -817,7 +817,7 @@ def test_two_stage_ring_matches_single():
              for r in range(2)]
     for p in procs:
         p.start()
-    out = q.get(timeout=200)
+    out = torch.tensor(q.get(timeout=200))
     for p in procs:
         p.join(timeout=60)
         assert p.exitcode == 0
