@@ -393,7 +393,7 @@ class FedinexRingModel(RingModel):
         mask = m.get("mask") or {}
         a = ops.attn_mod(q, kv.k[li], kv.v[li], pos, T, float(m["scale"]),
                          lens, slots, window=int(mask.get("size") or 0),
-                         keep=int(mask.get("keep_first") or 0))
+                         keep=int(mask.get("keep_first") or 0), wide=True)
         return lw.o(a)
 
     def _parallel(self, u, lw, lid, kv, pos, T, lens, slots, v_hop):
@@ -412,7 +412,8 @@ class FedinexRingModel(RingModel):
             conv_state=st["conv"], rot_freq=lw.rot_freq)
         ops.attn_mod(q, kv.k[li], kv.v[li], pos, T, float(lf["scale"]), lens,
                      slots, gate=p, gate_col=c["lg"],
-                     gate_scale=float(m["left_scale"]), out=y[:, :nl])
+                     gate_scale=float(m["left_scale"]), out=y[:, :nl],
+                     wide=True)
         ops.mlstm_heads(p, c["rq"], c["rk"], c["rv"], c["ri"], c["rf"],
                         lw.i_bias, lw.f_bias, float(rt["gate_cap"]),
                         rt["dim"] ** -0.5, st["S"], st["n"], st["m"], pos, T,

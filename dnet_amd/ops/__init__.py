@@ -517,7 +517,8 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
              sinks=None, window: int = 0, pool_k=None, pool_v=None,
              pool: int = 0, v_dim: int = 0, chunk: int = 0,
              sig_bias=None, keep: int = 0, gate=None, gate_col: int = 0,
-             gate_scale: float = 1.0, out=None) -> torch.Tensor:
+             gate_scale: float = 1.0, out=None,
+             wide: bool = False) -> torch.Tensor:
     """Causal attention against the cache with per-head temperature, tanh
     soft cap, logarithmic distance penalty and a sink in the softmax
     denominator (each optional). One entry point for decode (T=1) and
@@ -533,7 +534,9 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
     ``keep`` > 0 (with a window): the first ``keep`` keys stay visible beside
     the window. ``gate`` [B*T, ld]: head h's result times gate_scale *
     sigmoid(gate[row, gate_col + h]), before it is rounded. ``out``: a column
-    range of a wider zero-filled buffer for the result."""
+    range of a wider zero-filled buffer for the result. ``wide``: bf16
+    kernels keep the softmax weights to about 2^-17 in the value product (two
+    bf16 parts) instead of rounding them to bf16."""
     if keep:
         assert window and not pool and not chunk
     if sig_bias is not None:
@@ -586,7 +589,7 @@ def attn_mod(q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
                            pool_k if pool else None,
                            pool_v if pool else None, pool or 0, Dv,
                            chunk or 0, sig_bias, keep or 0, gate, gate_col,
-                           gate_scale)
+                           gate_scale, wide)
         return out
     return ref.attn_mod(q, kcache, vcache, pos, T, scale, lens, slots, temp,
                         softcap, dist_r1, dist_r2, sinks, window, pool_k,

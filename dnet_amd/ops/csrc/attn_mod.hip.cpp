@@ -25,6 +25,11 @@
 // sigmoid(gate[row, gate_col + h]) before it is rounded; the rows of the output
 // may be a column range of a wider buffer (row stride out_ld).
 //
+// Wide weights (wide): the matrix-core kernels hand the fp32 softmax weights to
+// the value product as two bf16 parts (the rounded weight and the rest), so that
+// no more than about 2^-17 of a weight is lost; the rows kernel keeps them fp32
+// anyway.
+//
 // Chunked visibility (chunk > 0): a query sees key j only inside its own block
 // of `chunk` positions, j >= (i / chunk) * chunk, blocks counted from position
 // 0. Sigmoid weights (sbias given): no softmax; a visible key weighs
@@ -477,7 +482,7 @@ __device__ __forceinline__ float fast_tanh(float x) {
   return 1.f - 2.f * __builtin_amdgcn_rcpf(__expf(2.f * x) + 1.f);
 }
 
-template <int DC, int NV>
+template <int DC, int NV, bool WIDE>
 __global__ __launch_bounds__(256) void attn_mod_mfma(
     const short* __restrict__ q, const short* __restrict__ kc,
     const short* __restrict__ vc, short* __restrict__ out,
@@ -644,10 +649,27 @@ __global__ __launch_bounds__(256) void attn_mod_mfma(
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // wave-local slab
     const bf16x8 pf =
         *reinterpret_cast<const bf16x8*>(&p_lds[wave][row * SP + hi * 8]);
+    bf16x8 rf;
+    if constexpr (WIDE) {
+      // what the rounding took off, through the same slab (a wave's LDS
+      // accesses stay in order)
+      asm volatile("" ::: "memory");
+#pragma unroll
+      for (int sub = 0; sub < 2; ++sub)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          p_lds[wave][(hi * 4 + r) * SP + sub * 16 + row] =
+              f2bits(p_val[sub][r] - bits2f(f2bits(p_val[sub][r])));
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+      rf = *reinterpret_cast<const bf16x8*>(&p_lds[wave][row * SP + hi * 8]);
+    }
 #pragma unroll
     for (int nn = 0; nn < NV; ++nn) {
       const bf16x8 vf = *reinterpret_cast<const bf16x8*>(
           &vt_lds[(nn * 16 + row) * SP + hi * 8]);
+      if constexpr (WIDE)
+        acc[nn] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(rf, vf, acc[nn], 0,
+                                                          0, 0);
       acc[nn] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf, vf, acc[nn], 0,
                                                         0, 0);
     }
@@ -685,7 +707,7 @@ __global__ __launch_bounds__(256) void attn_mod_mfma(
 // tiles, B); key tiles are dealt round robin to the splits and unnormalized
 // (acc, m, l) go to `partial` [B, Hq, splits, DV+2] for attn_mod_combine
 // (which also adds the sink). No pooled entries.
-template <int DC, int NV>
+template <int DC, int NV, bool WIDE>
 __global__ __launch_bounds__(256) void attn_mod_mfma_heads(
     const short* __restrict__ q, const short* __restrict__ kc,
     const short* __restrict__ vc, float* __restrict__ partial,
@@ -860,10 +882,27 @@ __global__ __launch_bounds__(256) void attn_mod_mfma_heads(
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // wave-local slab
     const bf16x8 pf =
         *reinterpret_cast<const bf16x8*>(&p_lds[wave][row * SP + hi * 8]);
+    bf16x8 rf;
+    if constexpr (WIDE) {
+      // what the rounding took off, through the same slab (a wave's LDS
+      // accesses stay in order)
+      asm volatile("" ::: "memory");
+#pragma unroll
+      for (int sub = 0; sub < 2; ++sub)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          p_lds[wave][(hi * 4 + r) * SP + sub * 16 + row] =
+              f2bits(p_val[sub][r] - bits2f(f2bits(p_val[sub][r])));
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+      rf = *reinterpret_cast<const bf16x8*>(&p_lds[wave][row * SP + hi * 8]);
+    }
 #pragma unroll
     for (int nn = 0; nn < NV; ++nn) {
       const bf16x8 vf = *reinterpret_cast<const bf16x8*>(
           &vt_lds[(nn * 16 + row) * SP + hi * 8]);
+      if constexpr (WIDE)
+        acc[nn] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(rf, vf, acc[nn], 0,
+                                                          0, 0);
       acc[nn] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf, vf, acc[nn], 0,
                                                         0, 0);
     }
@@ -918,7 +957,7 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
               int64_t v_dim, int64_t chunk,
               c10::optional<torch::Tensor> sig_bias, int64_t keep,
               c10::optional<torch::Tensor> gate, int64_t gate_col,
-              double gate_scale) {
+              double gate_scale, bool wide) {
   // no value cache: values = the first v_dim entries of the key rows
   const bool vshare = !vcache_opt.has_value();
   const torch::Tensor& vcache = vshare ? kcache : *vcache_opt;
@@ -1027,11 +1066,16 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
     float* part = partials->data_ptr<float>();
     const int GT = (G + 63) / 64;
     const dim3 hgrid((unsigned)ns, (unsigned)(Hkv * GT), (unsigned)B);
-#define AH(DCC, NVV)                                                         \
-  hipLaunchKernelGGL((attn_mod_mfma_heads<DCC, NVV>), hgrid, dim3(256), 0,   \
-                     stream, (const short*)q.data_ptr(),                     \
+#define AH_W(DCC, NVV, WW)                                                   \
+  hipLaunchKernelGGL((attn_mod_mfma_heads<DCC, NVV, WW>), hgrid, dim3(256),  \
+                     0, stream, (const short*)q.data_ptr(),                  \
                      (const short*)kcache.data_ptr(),                        \
                      (const short*)vcache.data_ptr(), part, ns, P)
+#define AH(DCC, NVV)                       \
+  do {                                     \
+    if (wide) AH_W(DCC, NVV, true);        \
+    else AH_W(DCC, NVV, false);            \
+  } while (0)
 #define AH_V(DCC)                          \
   do {                                     \
     if (DV <= 64) AH(DCC, 4);              \
@@ -1045,6 +1089,7 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
     else AH_V(8);
 #undef AH_V
 #undef AH
+#undef AH_W
     hipLaunchKernelGGL((attn_mod_combine<short>), dim3((unsigned)(B * Hq)),
                        dim3(64), 0, stream, part, (short*)out.data_ptr(), ns,
                        0, P);
@@ -1053,12 +1098,17 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
   // bf16 prompts: matrix-core kernel (head sizes padded to its tile classes)
   if (!f32 && T >= 16 && D % 8 == 0 && DV % 8 == 0) {
     const dim3 mgrid((unsigned)((T + 63) / 64), (unsigned)Hq, (unsigned)B);
-#define AM(DCC, NVV)                                                         \
-  hipLaunchKernelGGL((attn_mod_mfma<DCC, NVV>), mgrid, dim3(256), 0, stream, \
-                     (const short*)q.data_ptr(),                             \
+#define AM_W(DCC, NVV, WW)                                                   \
+  hipLaunchKernelGGL((attn_mod_mfma<DCC, NVV, WW>), mgrid, dim3(256), 0,     \
+                     stream, (const short*)q.data_ptr(),                     \
                      (const short*)kcache.data_ptr(),                        \
                      (const short*)vcache.data_ptr(), (short*)out.data_ptr(), \
                      P)
+#define AM(DCC, NVV)                       \
+  do {                                     \
+    if (wide) AM_W(DCC, NVV, true);        \
+    else AM_W(DCC, NVV, false);            \
+  } while (0)
 #define AM_V(DCC)                          \
   do {                                     \
     if (DV <= 64) AM(DCC, 4);              \
@@ -1072,6 +1122,7 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
     else AM_V(8);
 #undef AM_V
 #undef AM
+#undef AM_W
     return;
   }
   // split-KV (decode only): more workgroups when batch x kv heads is small

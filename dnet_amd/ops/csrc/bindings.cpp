@@ -130,7 +130,7 @@ void attn_mod(torch::Tensor q, torch::Tensor kcache,
               int64_t v_dim, int64_t chunk,
               c10::optional<torch::Tensor> sig_bias, int64_t keep,
               c10::optional<torch::Tensor> gate, int64_t gate_col,
-              double gate_scale);
+              double gate_scale, bool wide);
 void qkv_rope_append(torch::Tensor src, int64_t col0, int64_t nq, int64_t nkv,
                      int64_t d, int64_t dv, c10::optional<torch::Tensor> bias,
                      c10::optional<torch::Tensor> conv_w,

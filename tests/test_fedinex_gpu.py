@@ -129,6 +129,32 @@ def test_kept_tokens_and_output_gate(dt, G, Hkv, D, Dv, window, keep):
                                        want.float()[r], **_tol(dt))
 
 
+@pytest.mark.parametrize("G,Hkv,D,Dv", [(4, 2, 64, 64), (16, 1, 96, 128),
+                                        (32, 1, 200, 256), (2, 2, 128, 40)])
+def test_wide_weights(G, Hkv, D, Dv):
+    """The matrix-core kernels with two-part softmax weights: what is left is
+    the rounding of the result, well below what rounded weights add (prompt
+    kernel; grouped-heads decode kernel from 16 heads on)."""
+    torch.manual_seed(G * D)
+    B, S, T, Hq = 2, 300, 70, G * Hkv
+    dt = torch.bfloat16
+    k = torch.randn(B, Hkv, S, D, device=DEV).to(dt)
+    # values with a large common part: rounded weights no longer add up to one
+    v = (torch.randn(B, Hkv, S, Dv, device=DEV) * 0.05 + 3).to(dt)
+    for Tq in (T, 1):
+        pos = _i32([200, 37])
+        q = torch.randn(B * Tq, Hq * D, device=DEV).to(dt)
+        want = ref.attn_mod(q.cpu().float(), k.cpu().float(), v.cpu().float(),
+                            pos, Tq, D ** -0.5, window=90, keep=3)
+        err = []
+        for wide in (False, True):
+            out = ops.attn_mod(q, k, v, pos.to(DEV), Tq, D ** -0.5, window=90,
+                               keep=3, wide=wide)
+            err.append(float((out.cpu().float() - want).abs().mean()))
+        rounding = float((want.to(dt).float() - want).abs().mean())
+        assert err[1] <= 1.02 * rounding and err[1] <= err[0], (err, rounding)
+
+
 @pytest.mark.parametrize("dt", DTS)
 @pytest.mark.parametrize("H,d,dv,rank,T", [
     (3, 64, 32, 16, 37), (2, 20, 70, 5, 19), (1, 1, 1, 1, 9),
